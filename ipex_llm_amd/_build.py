@@ -81,10 +81,9 @@ def _cmd(src: str, obj: str):
             # some of them (profiles/gemv5_xm_forms_r6.txt)
             if os.path.basename(src) == "gemv_int4_xm.hip":
                 extra = ["-fno-slp-vectorize"]
-        if os.path.basename(src) in ("seqmix.hip", "ssm.hip", "maskattn.hip", "gatedmix.hip") or \
-                os.path.basename(src).startswith("blockmix_"):
-            # f32-exact kernels: no packed-f32 instruction forms
-            extra = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+        # f32 arithmetic as scalar instructions only: no packed-f32 forms in any kernel (the host pass does not know
+        # the feature and says so; harmless)
+        extra += ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
         return [HIPCC, f"--offload-arch={ARCH}", "-Wno-pass-failed", *extra, *common, "-c", src, "-o", obj]
     if "/cpu/" in src:
         return ["g++", *common, "-fopenmp", "-march=x86-64-v3", "-c", src, "-o", obj]
