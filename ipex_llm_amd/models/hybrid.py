@@ -56,6 +56,21 @@ Building blocks (each usable by any design that lists it in its layer specs):
   each result RMS-normed over the width, then their mean.
 * ``SoftmaxMoE``        experts whose weights are the softmax over the chosen
   router logits and multiply the experts' *outputs*; SiLU-gated experts.
+* ``MaskedAttention`` also takes a number per head that multiplies its scores
+  (``temp``) and an output gate with one number per head (``gate="head"``).
+* ``LightningAttention``  linear attention S' = decay_h S + k v^T, o = S'^T q with
+  a fixed decay per head, SiLU on q / k / v, one RMS norm over the joined heads,
+  a sigmoid output gate; f32 state.
+* ``GatedDelta``        gated delta rule: short convolutions with SiLU on q / k / v,
+  unit queries and keys, one decay and one step size per head,
+  S <- g S, S <- S + k (beta (v - S^T k))^T, o = S^T q; per-head RMS norm with a
+  SiLU gate; f32 state.
+* ``RealGatedLRU``      Griffin's recurrent block: a short convolution, gates from
+  block-diagonal matrices, S' = a S + sqrt(1 - a^2) i u element by element over
+  f32 state, multiplied by a tanh-GELU branch.
+* ``ScoredMoE``         experts weighed by their softmax score over *all* router
+  outputs, chosen by score + correction inside the best groups; some router
+  outputs may be identity experts (their result is the input itself).
 
 Block layouts.  ``pre_norm`` (``PreNormLayer``): x += mixer(norm1(x)),
 x += ff(norm2(x)) with vector RMS norms; each sublayer's result is added by
@@ -70,6 +85,10 @@ inputs are per-sequence state) and an optional token-side input afterwards.
 mixer's input shifted towards the previous token's:
 h = LN1(x), x += mixer(h + (h_prev - h) * mu) + ff(LN2(x)), then the token-side
 input.
+``sandwich`` (``SandwichLayer``): norms before and after every sublayer,
+x += N1b(mixer(N1(x))), x += N2b(ff(N2(x))) with statistics-free tanh norms
+(``DynTanh``); a sublayer's result is normed and added, and the next sublayer's
+norm formed, by one launch.
 The residual stream is f32 throughout; projections run in the model's
 activation dtype through the vendor GEMM, everything else in the kernels of
 ``ops/seqmix.py`` and ``ops/blockmix.py``.
@@ -92,6 +111,7 @@ from ..ops import gatedmix as GM
 from ..ops import maskattn as MA
 from ..ops import seqmix as SM
 from ..ops import ssm as SSM
+from ..ops import statemix as SX
 from .decoder import AttnMeta
 
 
@@ -152,7 +172,9 @@ class MaskedAttentionSpec:
     softcap: float = 0.0                    # > 0: score <- softcap tanh(score / softcap)
     sink_score: Optional[float] = None      # a sink of this fixed score (no tensor) instead of a learned one
     talk: bool = False                      # [H, H] mixing of the heads' weights after the softmax
-    out_gate: bool = False                  # element-wise sigmoid gate on the joined heads
+    out_gate: bool = False                  # sigmoid gate on the joined heads
+    gate: str = "element"                   # "element": one gate per value of the joined heads | "head": one per head
+    temp: bool = False                      # a learned number per head that multiplies its scores
 
 
 @dataclass
@@ -167,6 +189,31 @@ class GatedLinearAttentionSpec:
     vdim: int
     tau: float
     rank: int                               # of the low-rank decay projection
+
+
+@dataclass
+class LightningSpec:
+    heads: int
+    dim: int
+    vdim: int
+    decay: List[float]                      # one per head
+
+
+@dataclass
+class GatedDeltaSpec:
+    heads: int
+    kv_heads: int                           # query / key heads; head h reads h // (heads / kv_heads)
+    dim: int
+    vdim: int
+    taps: int                               # of the convolutions on q / k / v
+
+
+@dataclass
+class RealGatedLRUSpec:
+    width: int
+    blocks: int                             # of the block-diagonal gate matrices
+    taps: int
+    power: float = 8.0                      # log a = -power r softplus(lam)
 
 
 @dataclass
@@ -188,7 +235,9 @@ class MLSTMSpec:
 @dataclass
 class DenseFFSpec:
     ff: int
-    act: str = "gelu_tanh"                  # "gelu_tanh" | "relu" | "silu" on the gate rows
+    act: str = "gelu_tanh"                  # "gelu_tanh" | "relu" | "silu" on the gate rows | "clamp" (the clamped unit)
+    limit: float = float("inf")             # "clamp": g = min(gate, limit), u = clamp(up, -limit, limit),
+    alpha: float = 1.702                    #          g sigmoid(alpha g) (u + 1)
 
 
 @dataclass
@@ -221,6 +270,9 @@ class MoESpec:
     top: int
     expert: ExpertSpec = None
     shared: Optional[ExpertSpec] = None
+    identity: int = 0                       # the last router outputs beyond ``experts``: their result is the input
+    groups: int = 1                         # equal groups of neighbouring router outputs ...
+    keep: int = 1                           # ... of which the best ones take part in the choice
 
 
 @dataclass
@@ -248,8 +300,8 @@ class HybridSpec:
     bigram: Optional[BigramSpec] = None
     final_softcap: float = 0.0              # read by the engines' shared helpers
     logit_scale: float = 1.0                # the logits are multiplied by it
-    block: str = "post_norm"                # "post_norm" | "parallel" | "parallel2" | "pre_norm"
-    norm: str = "layer_norm"                # "layer_norm" | "rms_scalar" (one number) | "rms" (a vector)
+    block: str = "post_norm"                # "post_norm" | "parallel" | "parallel2" | "pre_norm" | "sandwich"
+    norm: str = "layer_norm"                # "layer_norm" | "rms_scalar" (one number) | "rms" (a vector) | "dyn_tanh"
     layer_scale: bool = False               # parallel blocks: per-coordinate scales on both sublayers' results
     canon_taps: int = 0                     # parallel blocks: taps of the convolution in front of the mixer (0: none)
     side_dim: int = 0                       # per-layer slice of the token-side table (0: none)
@@ -360,19 +412,22 @@ class MLSTM(nn.Module):
 
 
 class DenseFF(nn.Module):
-    """``W_down (act(W_gate h) * (W_up h))``"""
+    """``W_down (act(W_gate h) * (W_up h))``; ``act`` "clamp": ``W_down (g sigmoid(alpha g) (u + 1))`` with the gate
+    and up rows clamped by ``limit``"""
 
-    def __init__(self, w_gate, w_up, w_down, act: str = "gelu_tanh"):
+    def __init__(self, w_gate, w_up, w_down, act: str = "gelu_tanh", limit: float = float("inf"), alpha: float = 1.702):
         super().__init__()
-        if act not in SM.GLU_ACTS:
+        if act != "clamp" and act not in SM.GLU_ACTS:
             raise ValueError(f"unknown feed-forward activation {act!r}")
-        self.act = act
+        self.act, self.limit, self.alpha = act, limit, alpha
         self.w_gu = nn.Parameter(torch.cat([w_gate, w_up], 0).contiguous(), requires_grad=False)
         self.w_down = nn.Parameter(w_down, requires_grad=False)
 
     def forward(self, xa):
         if self.act == "gelu_tanh":
             return F.linear(SM.glu_gelu(F.linear(xa, self.w_gu)), self.w_down)
+        if self.act == "clamp":
+            return BM.linear(BM.glu_clamp(BM.linear(xa, self.w_gu), self.limit, self.alpha), self.w_down)
         return BM.linear(SM.glu_act(BM.linear(xa, self.w_gu), self.act), self.w_down)
 
 
@@ -428,11 +483,12 @@ class SSMMixer(nn.Module):
 class MaskedAttention(nn.Module):
     """``w_q`` [H d, W], ``w_k`` [G d, W], ``w_v`` [G dv, W] (``w_k`` / ``w_v`` None with ``kv_from``), biases or
     None, norm weights per ``qk_norm``, ``sink`` [H] or None, ``w_o`` [W, H dv]; optional ``conv`` = (q, k, v)
-    weights [channels, taps] (k / v None with ``kv_from``), ``talk`` [H, H], ``w_g`` [H dv, W]."""
+    weights [channels, taps] (k / v None with ``kv_from``), ``talk`` [H, H], ``w_g`` [H dv, W] ([H, W] with
+    ``gate="head"``), ``temp`` [H]."""
     cache_kind = "rows"
 
     def __init__(self, s: MaskedAttentionSpec, w_q, w_k, w_v, b_q, b_k, b_v, q_norm, k_norm, sink, w_o, conv=None,
-                 talk=None, w_g=None):
+                 talk=None, w_g=None, temp=None):
         super().__init__()
         if s.heads % s.kv_heads:
             raise ValueError("heads must be a multiple of kv_heads")
@@ -442,6 +498,8 @@ class MaskedAttention(nn.Module):
             raise ValueError("keep_first belongs to a window")
         if s.qk_norm not in ("none", "head", "whole"):
             raise ValueError(f"unknown qk_norm {s.qk_norm!r}")
+        if s.out_gate and s.gate not in ("head", "element"):
+            raise ValueError(f"unknown gate kind {s.gate!r}")
         self.s = s
         shared = s.kv_from is not None
         parts = [w_q] if shared else [w_q, w_k, w_v]
@@ -465,6 +523,7 @@ class MaskedAttention(nn.Module):
             sink = torch.full((s.heads,), float(s.sink_score), device=w_o.device)
         self.sink = nn.Parameter(sink.float().contiguous(), requires_grad=False) if sink is not None else None
         self.talk = nn.Parameter(talk.float().contiguous(), requires_grad=False) if s.talk else None
+        self.temp = nn.Parameter(temp.float().contiguous(), requires_grad=False) if s.temp else None
         self.w_o = nn.Parameter(w_o, requires_grad=False)
         self.table: Optional[torch.Tensor] = None
 
@@ -503,11 +562,11 @@ class MaskedAttention(nn.Module):
             v = y[:, (H + G) * d:(H + G) * d + G * dv].view(T, G, dv)
             rows = cache.rows[li]
             qf = MA.qkv_norm_rope_store(q, k, v, self.q_norm, self.k_norm, s.qk_norm == "whole", eps, table,
-                                        layout, pos, slots, rows)
+                                        layout, pos, slots, rows, temp=self.temp)
         else:
             rows = cache.rows[s.kv_from]
             qf = MA.qkv_norm_rope_store(q, None, None, self.q_norm, None, s.qk_norm == "whole", eps, table,
-                                        layout, pos, slots, None)
+                                        layout, pos, slots, None, temp=self.temp)
         o = MA.masked_attention(qf, rows, G, dv, meta.block_tables, meta.seq_of, pos, s.scale, s.mask.kind, s.mask.size,
                                 self.sink, meta.q_lens_host, meta.seq_lens_host, act, softcap=s.softcap,
                                 keep_first=s.mask.keep_first, talk=self.talk)
@@ -582,6 +641,130 @@ class GatedLinearAttention(nn.Module):
         return BM.linear(GM.head_rms_silu(o, self.norm, g, eps, y.dtype), self.w_o)
 
 
+class LightningAttention(nn.Module):
+    """``w_q`` / ``w_k`` [H d, W], ``w_v`` / ``w_g`` [H dv, W], ``norm`` [H dv], ``w_o`` [W, H dv]; the decays come
+    with the spec."""
+    cache_kind = "state"
+
+    def __init__(self, s: LightningSpec, w_q, w_k, w_v, w_g, norm, w_o):
+        super().__init__()
+        if len(s.decay) != s.heads:
+            raise ValueError("one decay per head")
+        self.s = s
+        self.w_in = nn.Parameter(torch.cat([w_q, w_k, w_v, w_g], 0).contiguous(), requires_grad=False)
+        self.b_in = None
+        self.decay = nn.Parameter(torch.tensor([float(v) for v in s.decay], dtype=torch.float32, device=w_o.device),
+                                  requires_grad=False)
+        self.norm = nn.Parameter(norm, requires_grad=False)
+        self.w_o = nn.Parameter(w_o, requires_grad=False)
+
+    def cache_spec(self):
+        s = self.s
+        return ("state", {"lightning": (s.heads, s.dim, s.vdim)})
+
+    def ensure_table(self, max_pos: int):
+        return None
+
+    def forward(self, xa, pos, slots, meta: AttnMeta, cache, li: int, eps: float):
+        return self.mix(BM.linear(xa, self.w_in), pos, slots, meta, cache, li, eps)
+
+    def mix(self, y, pos, slots, meta: AttnMeta, cache, li: int, eps: float):
+        s = self.s
+        T, H, d, dv = y.shape[0], s.heads, s.dim, s.vdim
+        nqk, nv = H * d, H * dv
+        q, k = y[:, :nqk].view(T, H, d), y[:, nqk:2 * nqk].view(T, H, d)
+        v, g = y[:, 2 * nqk:2 * nqk + nv].view(T, H, dv), y[:, 2 * nqk + nv:2 * nqk + 2 * nv]
+        o = SX.decay_scan(q, k, v, self.decay, cache.state[li]["lightning"], meta.cu_q, meta.state_slots, pos,
+                          meta.q_lens_host)
+        return BM.linear(SX.rms_sigmoid_gate(o.view(T, nv), self.norm, g, eps, y.dtype), self.w_o)
+
+
+class GatedDelta(nn.Module):
+    """``w_q`` / ``w_k`` [K d, W], ``w_v`` / ``w_g`` [H dv, W], ``w_a`` / ``w_b`` [H, W], ``conv`` = (q, k, v) weights
+    [channels, taps], ``a_log`` / ``dt_bias`` [H], ``norm`` [dv], ``w_o`` [W, H dv]."""
+    cache_kind = "state"
+
+    def __init__(self, s: GatedDeltaSpec, w_q, w_k, w_v, w_g, w_a, w_b, conv, a_log, dt_bias, norm, w_o):
+        super().__init__()
+        if s.heads % s.kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        if s.taps < 1 or s.taps > 16:
+            raise ValueError("1 <= conv taps <= 16")
+        self.s = s
+        self.n_qkv = int(w_q.shape[0] + w_k.shape[0] + w_v.shape[0])
+        self.w_in = nn.Parameter(torch.cat([w_q, w_k, w_v, w_g, w_a, w_b], 0).contiguous(), requires_grad=False)
+        self.b_in = None
+        self.conv = nn.Parameter(torch.cat(list(conv), 0).float().contiguous(), requires_grad=False)
+        self.rate = nn.Parameter(a_log.double().exp().float().contiguous(), requires_grad=False)
+        self.dt_bias = nn.Parameter(dt_bias.float().contiguous(), requires_grad=False)
+        self.norm = nn.Parameter(norm, requires_grad=False)
+        self.w_o = nn.Parameter(w_o, requires_grad=False)
+
+    def cache_spec(self):
+        s = self.s
+        return ("state", {"delta": (s.heads, s.dim, s.vdim), "conv": (s.taps - 1, self.n_qkv)})
+
+    def ensure_table(self, max_pos: int):
+        return None
+
+    def forward(self, xa, pos, slots, meta: AttnMeta, cache, li: int, eps: float):
+        return self.mix(BM.linear(xa, self.w_in), pos, slots, meta, cache, li, eps)
+
+    def mix(self, y, pos, slots, meta: AttnMeta, cache, li: int, eps: float):
+        s, st = self.s, cache.state[li]
+        T, H, K, d, dv = y.shape[0], s.heads, s.kv_heads, s.dim, s.vdim
+        n, nv = self.n_qkv, H * dv
+        g, a, b = y[:, n:n + nv], y[:, n + nv:n + nv + H], y[:, n + nv + H:n + nv + 2 * H]
+        u = SSM.conv_silu(y[:, :n], self.conv, None, st["conv"], meta.cu_q, meta.seq_of, meta.state_slots, pos,
+                          meta.q_lens_host)
+        q, k, v = u[:, :K * d].view(T, K, d), u[:, K * d:2 * K * d].view(T, K, d), u[:, 2 * K * d:].view(T, H, dv)
+        o = SX.delta_scan(q, k, v, a, b, self.rate, self.dt_bias, d ** -0.5, st["delta"], meta.cu_q, meta.state_slots,
+                          pos, meta.q_lens_host)
+        return BM.linear(GM.head_rms_silu(o, self.norm, g, eps, y.dtype), self.w_o)
+
+
+class RealGatedLRU(nn.Module):
+    """``w_x`` / ``w_y`` [width, W] with biases, ``conv_w`` [width, taps] (last column: the current token) with bias,
+    ``w_r`` / ``w_i`` [blocks, n, n] ([out, in]) with biases [blocks, n], ``lam`` [width], ``w_o`` [W, width]."""
+    cache_kind = "state"
+
+    def __init__(self, s: RealGatedLRUSpec, w_x, b_x, w_y, b_y, conv_w, conv_b, w_r, b_r, w_i, b_i, lam, w_o):
+        super().__init__()
+        if s.width % s.blocks:
+            raise ValueError("width must split into equal blocks")
+        if s.taps < 1 or s.taps > 16:
+            raise ValueError("1 <= conv taps <= 16")
+        self.s = s
+
+        def f32(t):
+            return nn.Parameter(t.float().reshape(-1).contiguous(), requires_grad=False)
+        self.w_in = nn.Parameter(torch.cat([w_x, w_y], 0).contiguous(), requires_grad=False)
+        self.b_in = nn.Parameter(torch.cat([b_x, b_y], 0).contiguous(), requires_grad=False)
+        self.conv_w = nn.Parameter(conv_w.float().contiguous(), requires_grad=False)
+        self.conv_b, self.b_r, self.b_i = f32(conv_b), f32(b_r), f32(b_i)
+        self.w_r = nn.Parameter(w_r.contiguous(), requires_grad=False)
+        self.w_i = nn.Parameter(w_i.contiguous(), requires_grad=False)
+        self.log_base = f32(-s.power * F.softplus(lam.double(), threshold=40.0))
+        self.w_o = nn.Parameter(w_o, requires_grad=False)
+
+    def cache_spec(self):
+        return ("state", {"lru": (self.s.width,), "lru_conv": (self.s.taps - 1, self.s.width)})
+
+    def ensure_table(self, max_pos: int):
+        return None
+
+    def forward(self, xa, pos, slots, meta: AttnMeta, cache, li: int, eps: float):
+        return self.mix(BM.linear(xa, self.w_in, self.b_in), pos, slots, meta, cache, li, eps)
+
+    def mix(self, y, pos, slots, meta: AttnMeta, cache, li: int, eps: float):
+        n, st = self.s.width, cache.state[li]
+        u = SSM.conv_silu(y[:, :n], self.conv_w, self.conv_b, st["lru_conv"], meta.cu_q, meta.seq_of, meta.state_slots,
+                          pos, meta.q_lens_host, act=False)
+        a, x = SX.rglru_gates(u, self.w_r, self.b_r, self.w_i, self.b_i, self.log_base)
+        o = SX.rglru_scan(a, x, y[:, n:], st["lru"], meta.cu_q, meta.state_slots, pos, meta.q_lens_host)
+        return BM.linear(o, self.w_o)
+
+
 class SideBySide(nn.Module):
     """Two mixers reading the same input: one projection launch over both mixers' input rows, then
     ``(rms_norm(left) * out_l + rms_norm(right) * out_r) / 2`` over the model width."""
@@ -624,11 +807,16 @@ class SideBySide(nn.Module):
             if hasattr(m, "table"):
                 m.table = v
 
-    def forward(self, xa, pos, slots, meta: AttnMeta, cache, li: int, eps: float):
+    def parts(self, xa, pos, slots, meta: AttnMeta, cache, li: int, eps: float) -> SX.PairMean:
+        """both mixers' results, their mean still to be formed (by the launch that adds it to the residual stream)"""
         y = BM.linear(xa, self.w_in, self.b_in)
         a = self.left.mix(y[:, :self.n_left], pos, slots, meta, cache, li, eps)
         b = self.right.mix(y[:, self.n_left:], pos, slots, meta, cache, li, eps)
-        return GM.rms_pair_mean(a, b, self.out_l, self.out_r, eps, xa.dtype)
+        return SX.PairMean(a, b, self.out_l, self.out_r, eps)
+
+    def forward(self, xa, pos, slots, meta: AttnMeta, cache, li: int, eps: float):
+        p = self.parts(xa, pos, slots, meta, cache, li, eps)
+        return GM.rms_pair_mean(p.a, p.b, p.wa, p.wb, eps, xa.dtype)
 
 
 class GroupedAttention(nn.Module):
@@ -722,6 +910,34 @@ class SoftmaxMoE(nn.Module):
         idx, wts = BM.moe_route(F.linear(xa.float() if x32 is None else x32, self.router), s.top, "softmax")
         y = BM.moe_experts(xa, idx, wts, self.w_gu, self.w_down, float("inf"), 1.0, 0.0, "output")
         return y, None
+
+
+class ScoredMoE(nn.Module):
+    """``router`` [experts + identity, W], ``correction`` [experts + identity] or None, ``w_gu`` [E, 2 ff, W] (every
+    expert's gate rows, then its up rows), ``w_down`` [E, W, ff].  Scores are the softmax of f32 logits over all router
+    outputs; the choice goes by score + correction inside the best groups, the weights are the plain scores and
+    multiply the experts' *outputs*; experts ``W_down (silu(W_gate h) * (W_up h))``, identity experts ``h``."""
+
+    def __init__(self, s: MoESpec, router, correction, w_gu, w_down):
+        super().__init__()
+        n = s.experts + s.identity
+        if s.groups < 1 or n % s.groups or not 1 <= s.keep <= s.groups or not 1 <= s.top <= s.keep * (n // s.groups):
+            raise ValueError("router: equal groups, 1 <= keep <= groups, 1 <= top <= experts of the kept groups")
+        self.s = s
+        self.router = nn.Parameter(router.float().contiguous(), requires_grad=False)
+        self.correction = nn.Parameter(correction.float().contiguous(), requires_grad=False) if correction is not None else None
+        self.w_gu = nn.Parameter(w_gu.contiguous(), requires_grad=False)
+        self.w_down = nn.Parameter(w_down.contiguous(), requires_grad=False)
+
+    def parts(self, xa) -> SX.ExpertSum:
+        """the chosen experts' weighted results, their sum still to be formed"""
+        s = self.s
+        idx, wts = SX.route_groups(F.linear(xa.float(), self.router), self.correction, s.top, s.groups, s.keep)
+        rows = BM.moe_expert_rows(xa, idx, wts, self.w_gu, self.w_down, float("inf"), 1.0, 0.0, "output", s.identity)
+        return SX.ExpertSum(rows, idx, wts, xa, s.experts)
+
+    def forward(self, xa, x32=None):
+        return self.parts(xa).value(), None
 
 
 class TokenSide(nn.Module):
@@ -852,6 +1068,46 @@ class TwoNormParallelLayer(nn.Module):
         return xa
 
 
+class DynTanh(nn.Module):
+    """``tanh(alpha x) w + b``: a norm without statistics; ``alpha`` one number, ``w`` / ``b`` [W]"""
+
+    def __init__(self, alpha, w, b):
+        super().__init__()
+        self.alpha = nn.Parameter(alpha.float().reshape(1).contiguous(), requires_grad=False)
+        self.w = nn.Parameter(w.float().contiguous(), requires_grad=False)
+        self.b = nn.Parameter(b.float().contiguous(), requires_grad=False)
+
+    @property
+    def args(self) -> SX.Norm:
+        return self.alpha, self.w, self.b
+
+
+class SandwichLayer(nn.Module):
+    """x += post1(mixer(pre1(x)));  x += post2(ff(pre2(x))).  The layer receives ``pre1(x)`` and returns the next
+    layer's (the model's final norm after the last one): the launch that norms and adds a sublayer's result also
+    forms the norm in front of the next sublayer."""
+
+    def __init__(self, mixer: nn.Module, pre1: DynTanh, post1: DynTanh, mlp: Optional[nn.Module] = None,
+                 pre2: Optional[DynTanh] = None, post2: Optional[DynTanh] = None):
+        super().__init__()
+        self.mixer, self.mlp = mixer, mlp
+        self.pre1, self.post1, self.pre2, self.post2 = pre1, post1, pre2, post2
+
+    def cache_specs(self):
+        return _spec_list(self.mixer.cache_spec())
+
+    def forward(self, x, h, ids, pos, slots, meta, cache, li: int, model):
+        s, act = model.spec, model.dtype
+        after = (model.layers[li + 1].pre1 if li + 1 < len(model.layers) else model.norm).args
+        run = getattr(self.mixer, "parts", self.mixer)
+        y = run(h, pos, slots, meta, cache, li, s.norm_eps)
+        if self.mlp is None:
+            return SX.add_normed_(x, y, self.post1.args, after, act)
+        h = SX.add_normed_(x, y, self.post1.args, self.pre2.args, act)
+        y = getattr(self.mlp, "parts", self.mlp)(h)
+        return SX.add_normed_(x, y, self.post2.args, after, act)
+
+
 # name -> (spec class, module class): a design's config reader maps its layer
 # types onto these
 MIXERS: Dict[str, tuple] = {"latent_attention": (LatentAttentionSpec, LatentAttention), "mlstm": (MLSTMSpec, MLSTM),
@@ -859,6 +1115,9 @@ MIXERS: Dict[str, tuple] = {"latent_attention": (LatentAttentionSpec, LatentAtte
                             "ssm": (SSMSpec, SSMMixer), "masked_attention": (MaskedAttentionSpec, MaskedAttention),
                             "mingru": (MinGRUSpec, MinGRU),
                             "gated_linear_attention": (GatedLinearAttentionSpec, GatedLinearAttention),
+                            "lightning": (LightningSpec, LightningAttention),
+                            "gated_delta": (GatedDeltaSpec, GatedDelta),
+                            "real_gated_lru": (RealGatedLRUSpec, RealGatedLRU),
                             "side_by_side": (SideBySideSpec, SideBySide)}
 
 
@@ -868,7 +1127,7 @@ class HybridCausalLM(nn.Module):
     native_lib = "seqmix"           # the kernels it needs (ops.require_seqmix)
 
     def __init__(self, spec: HybridSpec, embed: torch.Tensor, bigram: Optional[torch.Tensor],
-                 layers: List[nn.Module], final_norm: torch.Tensor, head: torch.Tensor, dtype=torch.bfloat16,
+                 layers: List[nn.Module], final_norm, head: Optional[torch.Tensor], dtype=torch.bfloat16,
                  side_embed: Optional[torch.Tensor] = None):
         super().__init__()
         self.spec, self.dtype = spec, dtype
@@ -876,7 +1135,7 @@ class HybridCausalLM(nn.Module):
         self.bigram = nn.Parameter(bigram, requires_grad=False) if bigram is not None else None
         self.side_embed = nn.Parameter(side_embed, requires_grad=False) if side_embed is not None else None
         self.layers = nn.ModuleList(layers)
-        self.norm = nn.Parameter(final_norm, requires_grad=False)
+        self.norm = final_norm if isinstance(final_norm, nn.Module) else nn.Parameter(final_norm, requires_grad=False)
         # a tied head (head None) is the embedding table itself
         self.lm_head = nn.Parameter(head, requires_grad=False) if head is not None else self.embed_tokens
         self.tp_group = None
@@ -885,7 +1144,7 @@ class HybridCausalLM(nn.Module):
 
     @property
     def device(self):
-        return self.norm.device
+        return self.embed_tokens.device
 
     @property
     def has_state(self) -> bool:
@@ -948,7 +1207,10 @@ class HybridCausalLM(nn.Module):
         else:
             x = F.embedding(ids, self.embed_tokens).float()
         pre = s.block == "pre_norm"         # ``xa`` is then the last sublayer's result, still to be added to x
-        xa = None if pre else (x if act == torch.float32 else x.to(act))
+        if s.block == "sandwich":           # ``xa`` is the norm of x in front of the next sublayer
+            xa = SX.dyn_tanh(x, (self.layers[0].pre1 if len(self.layers) else self.norm).args, act)
+        else:
+            xa = None if pre else (x if act == torch.float32 else x.to(act))
         for li, L in enumerate(self.layers):
             xa = L(x, xa, ids, pos, slots, meta, cache, li, self)
             if self.capture_layers is not None:
@@ -957,8 +1219,10 @@ class HybridCausalLM(nn.Module):
             return x.add_(xa.float()) if pre and xa is not None else x
         if logits_idx is not None:
             x = x.index_select(0, logits_idx)
-            xa = xa.index_select(0, logits_idx) if pre and xa is not None else xa
-        if pre:
+            xa = xa.index_select(0, logits_idx) if xa is not None else xa
+        if s.block == "sandwich":
+            xn = xa                         # the last layer formed the final norm
+        elif pre:
             xn = BM.add_rms_norm_rows_(x, xa, self.norm, s.norm_eps, act)
         elif s.norm == "layer_norm":
             xn = SM.layer_norm_f32(x, self.norm, s.norm_eps, act)

@@ -20,6 +20,7 @@ NATIVE_ARCHITECTURES = {
     "Masezen": "ipex_llm_amd.models.masezen",
     "Vogolix": "ipex_llm_amd.models.vogolix",
     "Zoguzen": "ipex_llm_amd.models.zoguzen",
+    "Sudosun": "ipex_llm_amd.models.sudosun",
 }
 
 

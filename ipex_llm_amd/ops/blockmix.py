@@ -24,7 +24,8 @@ import torch.nn.functional as F
 from .seqmix import native, _mm_f32
 
 __all__ = ["linear", "rms_norm_rows", "add_rms_norm_rows_", "canon_conv", "norm_canon", "qk_norm_rope_store", "talk_attention", "relu_sq", "glu_clamp",
-           "residual_add_scaled_", "side_gate", "add_rms_norm_", "moe_route", "moe_experts"]
+           "residual_add_scaled_", "side_gate", "add_rms_norm_", "moe_route", "moe_experts",
+           "moe_expert_rows"]
 
 
 def _ops():
@@ -366,13 +367,24 @@ def moe_experts(h: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor, w_gu: tor
     ``W_down (g sigmoid(alpha g) (u + up_shift))`` with g = min(gate, limit),
     u = clamp(up, -limit, limit) (``limit`` may be infinite; alpha = 1,
     up_shift = 0: the SiLU-gated unit).  Returns f32 [T, W]."""
+    rows = moe_expert_rows(h, idx, wts, w_gu, w_down, limit, alpha, up_shift, weigh)
+    return rows[:, 0] if idx.shape[1] == 1 else rows.sum(1)
+
+
+def moe_expert_rows(h: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor, w_gu: torch.Tensor, w_down: torch.Tensor,
+                    limit: float, alpha: float = 1.702, up_shift: float = 1.0, weigh: str = "input",
+                    identity: int = 0) -> torch.Tensor:
+    """The terms of ``moe_experts`` before their sum: f32 [T, top, W].  With
+    ``identity``, indices E .. E + identity - 1 name identity experts: their rows
+    are left as they are (any content), the caller adds ``w h`` for them."""
     T, W = h.shape
     top = idx.shape[1]
     if weigh not in ("input", "output"):
         raise ValueError(f"unknown weighing {weigh!r}")
     if native(h):
-        return _ops().bm_moe_experts(h.contiguous(), idx, wts, w_gu, w_down, limit, alpha, up_shift, weigh == "output")
-    out = torch.zeros(T, W, dtype=torch.float32, device=h.device)
+        return _ops().bm_moe_expert_rows(h.contiguous(), idx, wts, w_gu, w_down, limit, alpha, up_shift,
+                                         weigh == "output", identity)
+    out = torch.zeros(T, top, W, dtype=torch.float32, device=h.device)
     E = w_gu.shape[0]
     I = w_gu.shape[1] // 2
     for k in range(top):
@@ -386,5 +398,5 @@ def moe_experts(h: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor, w_gu: tor
             u = gu[..., I:].float().clamp(-limit, limit)
             y = (g * torch.sigmoid(alpha * g) * (u + up_shift)).to(h.dtype)
             r = F.linear(y, w_down[e]).float()
-            out[sel] += r * wts[sel, k:k + 1] if weigh == "output" else r
+            out[sel, k] = r * wts[sel, k:k + 1] if weigh == "output" else r
     return out

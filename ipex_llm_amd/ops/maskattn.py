@@ -64,7 +64,7 @@ def _turn(x: torch.Tensor, cs: torch.Tensor, layout: str) -> torch.Tensor:
 def qkv_norm_rope_store(q: torch.Tensor, k: Optional[torch.Tensor], v: Optional[torch.Tensor],
                         q_norm: Optional[torch.Tensor], k_norm: Optional[torch.Tensor], whole: bool, eps: float,
                         table: Optional[torch.Tensor], layout: str, pos: torch.Tensor, slots: torch.Tensor,
-                        rows: Optional[torch.Tensor]) -> torch.Tensor:
+                        rows: Optional[torch.Tensor], temp: Optional[torch.Tensor] = None) -> torch.Tensor:
     """RMS norm and rotary positions of ``q`` [T, H, d] and ``k`` [T, G, d]
     (strided views allowed), and one cache row per token.
 
@@ -76,11 +76,12 @@ def qkv_norm_rope_store(q: torch.Tensor, k: Optional[torch.Tensor], v: Optional[
     rotation.  When ``k`` is given, ``[keys (normed, rotated) | v as projected]``
     is written at row index ``slots`` of the paged pool ``rows``
     [blocks, bs, G d + G dv]; a layer that reads another layer's rows passes
-    ``k = v = rows = None``.  Returns the queries f32 [T, H, d]."""
+    ``k = v = rows = None``.  ``temp`` f32 [H]: head h's queries (and so its scores) are multiplied by ``temp[h]``.
+    Returns the queries f32 [T, H, d]."""
     T, H, d = q.shape
     if native(q):
         return _ops().ma_qkv_norm_rope_store(q, k, v, q_norm, k_norm, whole, eps, table, LAYOUTS[layout], pos, slots,
-                                             rows)
+                                             rows, temp)
     cs = table[pos.long()][:, None] if table is not None else None
 
     def prep(x, w):
@@ -99,7 +100,7 @@ def qkv_norm_rope_store(q: torch.Tensor, k: Optional[torch.Tensor], v: Optional[
         kf = prep(k, k_norm)
         flat = rows.view(-1, rows.shape[-1])
         flat.index_copy_(0, slots.long(), torch.cat([kf.reshape(T, -1), v.float().reshape(T, -1)], -1).to(rows.dtype))
-    return qf.contiguous()
+    return (qf * temp.float()[:, None] if temp is not None else qf).contiguous()
 
 
 # GPU paths by portion: decoded tokens and short pieces run the one-pass kernel, a workgroup per (token, key head).
@@ -332,7 +333,9 @@ def _bmm_f32_ok(dtype) -> bool:
 
 def sigmoid_gate(o: torch.Tensor, gate_pre: torch.Tensor) -> torch.Tensor:
     """``o * sigmoid(gate_pre)`` element by element (f32 math), o's dtype;
-    ``gate_pre`` may be a strided view of a projection's result."""
+    ``gate_pre`` may be a strided view of a projection's result.  A gate of
+    fewer columns ([T, H] beside o [T, H dv]) holds one number per head."""
     if native(o):
         return _ops().ma_sigmoid_gate(o.contiguous(), gate_pre)
-    return (o.float() * torch.sigmoid(gate_pre.float())).to(o.dtype)
+    g = torch.sigmoid(gate_pre.float()).repeat_interleave(o.shape[1] // gate_pre.shape[1], 1)
+    return (o.float() * g).to(o.dtype)
