@@ -69,8 +69,9 @@ void talk_softmax(bool bf16, float* sc, const int64_t* pos, int H, float scale, 
 // ---- experts (blockmix_moe.hip)
 // mode 0: the largest sigmoid(z) win and are the weights; 1: the largest logits win, softmax over the winners (top <= 64)
 void moe_route(const float* z, int T, int E, int top, int32_t* idx, float* w, int mode, hipStream_t st);
-// off int32 [E + 1], sorted int32 [P]: pair ids (token * top + k) grouped by expert
-void moe_align(const int32_t* idx, int P, int E, int32_t* off, int32_t* sorted, hipStream_t st);
+// off int32 [E + 1], sorted int32 [P]: pair ids (token * top + k) grouped by expert; pairs of the ``ident`` identity
+// experts E .. E + ident - 1 are left out
+void moe_align(const int32_t* idx, int P, int E, int ident, int32_t* off, int32_t* sorted, hipStream_t st);
 // y [P, ff] (sorted order) = glu(W_gu[e] (w_p h_token)), glu = g sigmoid(alpha g) (u + up_shift) with the clamps;
 // weigh_out: the input is h_token itself (the routing weight multiplies the result of moe_down instead)
 void moe_glu(bool bf16, const void* h, const int32_t* off, const int32_t* sorted, const float* wts, int top,

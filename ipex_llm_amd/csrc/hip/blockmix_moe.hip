@@ -87,14 +87,16 @@ __global__ void __launch_bounds__(64) moe_route_k(const float* __restrict__ z, i
   if (SOFTMAX && lane < top) w[t * top + lane] = mine / den;
 }
 
-__global__ void __launch_bounds__(1024) moe_align_k(const int32_t* __restrict__ idx, int P, int E, int32_t* __restrict__ off,
-                                                   int32_t* __restrict__ sorted) {
+// pairs whose index is E .. E + ident - 1 (identity experts) get no place
+__global__ void __launch_bounds__(1024) moe_align_k(const int32_t* __restrict__ idx, int P, int E, int ident,
+                                                   int32_t* __restrict__ off, int32_t* __restrict__ sorted) {
   extern __shared__ int cnt[];                       // [E] counters, then [E] cursors
   int* cur = cnt + E;
   for (int e = threadIdx.x; e < E; e += blockDim.x) cnt[e] = 0;
   __syncthreads();
   for (int p = threadIdx.x; p < P; p += blockDim.x) {
     int e = idx[p];
+    if (e >= E && e < E + ident) continue;
     e = e < 0 ? 0 : (e >= E ? E - 1 : e);
     atomicAdd(&cnt[e], 1);
   }
@@ -111,6 +113,7 @@ __global__ void __launch_bounds__(1024) moe_align_k(const int32_t* __restrict__ 
   __syncthreads();
   for (int p = threadIdx.x; p < P; p += blockDim.x) {
     int e = idx[p];
+    if (e >= E && e < E + ident) continue;
     e = e < 0 ? 0 : (e >= E ? E - 1 : e);
     sorted[atomicAdd(&cur[e], 1)] = p;
   }
@@ -360,8 +363,8 @@ void moe_route(const float* z, int T, int E, int top, int32_t* idx, float* w, in
   else moe_route_k<false><<<T, 64, 0, st>>>(z, E, top, idx, w);
 }
 
-void moe_align(const int32_t* idx, int P, int E, int32_t* off, int32_t* sorted, hipStream_t st) {
-  moe_align_k<<<1, 1024, (size_t)2 * E * sizeof(int), st>>>(idx, P, E, off, sorted);
+void moe_align(const int32_t* idx, int P, int E, int ident, int32_t* off, int32_t* sorted, hipStream_t st) {
+  moe_align_k<<<1, 1024, (size_t)2 * E * sizeof(int), st>>>(idx, P, E, ident, off, sorted);
 }
 
 void moe_glu(bool bf16, const void* h, const int32_t* off, const int32_t* sorted, const float* wts, int top,

@@ -21,7 +21,7 @@ enum Layout { kPairs = 0, kHalf = 1 };     // rotary pairs (2 i, 2 i + 1) or (i,
 void qkv_norm_rope_store(bool in_bf16, bool bf16, const void* q, int64_t q_ld, const void* k, int64_t k_ld,
                          const void* v, int64_t v_ld, const void* qn, const void* kn, bool whole, float eps,
                          const float* table, int max_pos, int dims, int layout, const int64_t* pos, const int64_t* slots,
-                         void* rows, int64_t num_rows, float* qo, int T, int H, int G, int d, int dv, hipStream_t st);
+                         void* rows, int64_t num_rows, float* qo, const float* temp, int T, int H, int G, int d, int dv, hipStream_t st);
 
 // dynamic LDS of the attention launch (waves and heads per workgroup out); < 0: these sizes do not fit
 int masked_attention_plan(bool bf16, int rep, int d, int dv, int* nw, int* hb);
@@ -52,7 +52,7 @@ void talk_mix(bool bf16, const float* w, const float* talk, int64_t pieces, int 
               float* out32, hipStream_t st);
 
 // o[t, c] *= sigmoid(g[t, c]); g rows of g_ld elements
-void sigmoid_gate(bool bf16, void* o, const void* g, int64_t g_ld, int64_t T, int C, hipStream_t st);
+void sigmoid_gate(bool bf16, void* o, const void* g, int64_t g_ld, int64_t T, int C, int per, hipStream_t st);
 
 }  // namespace ma
 }  // namespace illm

@@ -81,8 +81,8 @@ __global__ void __launch_bounds__(1024) qkv_store_k(const EI* __restrict__ q, in
                                                   const E* __restrict__ qn, const E* __restrict__ kn, bool whole,
                                                   float eps, const float* __restrict__ table, int dims, int layout,
                                                   const int64_t* __restrict__ pos, const int64_t* __restrict__ slots,
-                                                  E* __restrict__ rows, float* __restrict__ qo, int H, int G, int d,
-                                                  int dv) {
+                                                  E* __restrict__ rows, float* __restrict__ qo,
+                                                  const float* __restrict__ temp, int H, int G, int d, int dv) {
   extern __shared__ float hs[];                                     // [H + G] (+ 2 totals)
   const int64_t t = blockIdx.x;
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, NW = blockDim.x >> 6;
@@ -138,7 +138,7 @@ __global__ void __launch_bounds__(1024) qkv_store_k(const EI* __restrict__ q, in
       const float c = cs[2 * pi], s = cs[2 * pi + 1];
       val = first ? val * c - other * s : val * c + other * s;
     }
-    if (isq) qo[(t * H + head) * d + i] = val;
+    if (isq) qo[(t * H + head) * d + i] = temp ? val * temp[head] : val;
     else stf(row + head * d + i, val);
   }
   if (k)
@@ -512,13 +512,14 @@ __global__ void __launch_bounds__(256) chunk_softmax_k(float* __restrict__ sc, i
   }
 }
 
+// per: consecutive values that share a gate
 template <typename E>
 __global__ void __launch_bounds__(256) sigmoid_gate_k(E* __restrict__ o, const E* __restrict__ g, int64_t g_ld, int64_t n,
-                                                     int C) {
+                                                     int C, int per) {
   for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (int64_t)gridDim.x * blockDim.x) {
     const int64_t t = i / C;
     const int c = (int)(i - t * C);
-    stf(o + i, ldf(o + i) / (1.0f + expf(-ldf(g + t * g_ld + c))));
+    stf(o + i, ldf(o + i) / (1.0f + expf(-ldf(g + t * g_ld + (per > 1 ? c / per : c)))));
   }
 }
 
@@ -534,7 +535,8 @@ int tile_row(int d, int dv) {
 void qkv_norm_rope_store(bool in_bf16, bool bf16, const void* q, int64_t q_ld, const void* k, int64_t k_ld,
                          const void* v, int64_t v_ld, const void* qn, const void* kn, bool whole, float eps,
                          const float* table, int max_pos, int dims, int layout, const int64_t* pos, const int64_t* slots,
-                         void* rows, int64_t num_rows, float* qo, int T, int H, int G, int d, int dv, hipStream_t st) {
+                         void* rows, int64_t num_rows, float* qo, const float* temp, int T, int H, int G, int d, int dv,
+                         hipStream_t st) {
   (void)max_pos;
   (void)num_rows;
   if (T <= 0) return;
@@ -544,8 +546,8 @@ void qkv_norm_rope_store(bool in_bf16, bool bf16, const void* q, int64_t q_ld, c
   const int nt = T > 64 ? 256 : (vals >= 1024 ? 1024 : (int)((vals + 63) / 64 * 64));
 #define MA_STORE(EI, E)                                                                                                 \
   qkv_store_k<EI, E><<<T, nt, lds, st>>>((const EI*)q, q_ld, (const EI*)k, k_ld, (const EI*)v, v_ld, (const E*)qn,      \
-                                         (const E*)kn, whole, eps, table, dims, layout, pos, slots, (E*)rows, qo, H, G, \
-                                         d, dv)
+                                         (const E*)kn, whole, eps, table, dims, layout, pos, slots, (E*)rows, qo, temp, \
+                                         H, G, d, dv)
   if (bf16 && in_bf16) MA_STORE(__bf16, __bf16);
   else if (bf16) MA_STORE(float, __bf16);
   else MA_STORE(float, float);
@@ -646,12 +648,12 @@ void talk_mix(bool bf16, const float* w, const float* talk, int64_t pieces, int 
   else talk_mix_k<float><<<grid, 64, lds, st>>>(w, talk, Lq, L, G, rep, (float*)nullptr, out32);
 }
 
-void sigmoid_gate(bool bf16, void* o, const void* g, int64_t g_ld, int64_t T, int C, hipStream_t st) {
+void sigmoid_gate(bool bf16, void* o, const void* g, int64_t g_ld, int64_t T, int C, int per, hipStream_t st) {
   const int64_t n = T * C;
   if (n <= 0) return;
   const int blocks = (int)((n + 255) / 256 > 65535 ? 65535 : (n + 255) / 256);
-  if (bf16) sigmoid_gate_k<__bf16><<<blocks, 256, 0, st>>>((__bf16*)o, (const __bf16*)g, g_ld, n, C);
-  else sigmoid_gate_k<float><<<blocks, 256, 0, st>>>((float*)o, (const float*)g, g_ld, n, C);
+  if (bf16) sigmoid_gate_k<__bf16><<<blocks, 256, 0, st>>>((__bf16*)o, (const __bf16*)g, g_ld, n, C, per);
+  else sigmoid_gate_k<float><<<blocks, 256, 0, st>>>((float*)o, (const float*)g, g_ld, n, C, per);
 }
 
 }  // namespace ma

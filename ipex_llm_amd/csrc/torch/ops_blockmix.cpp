@@ -370,40 +370,40 @@ std::tuple<Tensor, Tensor> bm_moe_route(const Tensor& z, int64_t top, int64_t mo
   return {idx, w};
 }
 
-Tensor bm_moe_experts(const Tensor& h, const Tensor& idx, const Tensor& wts, const Tensor& w_gu, const Tensor& w_down,
-                      double limit, double alpha, double up_shift, bool weigh_out) {
+Tensor bm_moe_expert_rows(const Tensor& h, const Tensor& idx, const Tensor& wts, const Tensor& w_gu, const Tensor& w_down,
+                      double limit, double alpha, double up_shift, bool weigh_out, int64_t identity) {
   c10::DeviceGuard g(h.device());
-  TORCH_CHECK(h.is_cuda() && h.dim() == 2 && is_act(h) && h.is_contiguous(), "bm_moe_experts: h [T, W] contiguous");
+  TORCH_CHECK(h.is_cuda() && h.dim() == 2 && is_act(h) && h.is_contiguous(), "bm_moe_expert_rows: h [T, W] contiguous");
   const int64_t T = h.size(0), W = h.size(1);
   TORCH_CHECK(idx.is_cuda() && idx.scalar_type() == at::kInt && idx.is_contiguous() && idx.dim() == 2 &&
                   idx.size(0) == T && idx.size(1) >= 1,
-              "bm_moe_experts: idx int32 [T, top]");
+              "bm_moe_expert_rows: idx int32 [T, top]");
   const int64_t top = idx.size(1), P = T * top;
   TORCH_CHECK(wts.is_cuda() && wts.scalar_type() == at::kFloat && wts.is_contiguous() && wts.numel() == P,
-              "bm_moe_experts: weights f32 [T, top]");
+              "bm_moe_expert_rows: weights f32 [T, top]");
   TORCH_CHECK(w_gu.is_cuda() && w_gu.dim() == 3 && w_gu.scalar_type() == h.scalar_type() && w_gu.is_contiguous() &&
                   w_gu.size(2) == W && w_gu.size(1) % 2 == 0,
-              "bm_moe_experts: w_gu [E, 2 ff, W] of h's dtype");
+              "bm_moe_expert_rows: w_gu [E, 2 ff, W] of h's dtype");
   const int64_t E = w_gu.size(0), ff = w_gu.size(1) / 2;
-  TORCH_CHECK(E <= 1024, "bm_moe_experts: at most 1024 experts");
+  TORCH_CHECK(E <= 1024, "bm_moe_expert_rows: at most 1024 experts");
+  TORCH_CHECK(identity >= 0 && identity <= 1 << 20, "bm_moe_expert_rows: identity experts");
   TORCH_CHECK(w_down.is_cuda() && w_down.dim() == 3 && w_down.scalar_type() == h.scalar_type() &&
                   w_down.is_contiguous() && w_down.size(0) == E && w_down.size(1) == W && w_down.size(2) == ff,
-              "bm_moe_experts: w_down [E, W, ff] of h's dtype");
+              "bm_moe_expert_rows: w_down [E, W, ff] of h's dtype");
   auto iopt = h.options().dtype(at::kInt);
   Tensor off = at::empty({E + 1}, iopt), sorted = at::empty({P}, iopt);
   Tensor y = at::empty({P, ff}, h.options());
   Tensor out = at::empty({P, W}, h.options().dtype(at::kFloat));
-  if (P == 0) return out.view({T, W});
+  if (P == 0) return out.view({T, top, W});
   auto st = stream();
-  illm::bm::moe_align(idx.data_ptr<int32_t>(), (int)P, (int)E, off.data_ptr<int32_t>(), sorted.data_ptr<int32_t>(), st);
+  illm::bm::moe_align(idx.data_ptr<int32_t>(), (int)P, (int)E, (int)identity, off.data_ptr<int32_t>(), sorted.data_ptr<int32_t>(), st);
   illm::bm::moe_glu(bf(h), h.data_ptr(), off.data_ptr<int32_t>(), sorted.data_ptr<int32_t>(), wts.data_ptr<float>(),
                     (int)top, w_gu.data_ptr(), y.data_ptr(), (int)P, (int)E, (int)ff, (int)W, (float)limit,
                     (float)alpha, (float)up_shift, weigh_out, st);
   illm::bm::moe_down(bf(h), y.data_ptr(), off.data_ptr<int32_t>(), sorted.data_ptr<int32_t>(), w_down.data_ptr(),
                      out.data_ptr<float>(), (int)P, (int)E, (int)ff, (int)W, weigh_out ? wts.data_ptr<float>() : nullptr,
                      st);
-  if (top == 1) return out;
-  return out.view({T, top, W}).sum(1);
+  return out.view({T, top, W});
 }
 
 }  // namespace
@@ -432,8 +432,8 @@ TORCH_LIBRARY_FRAGMENT(ipex_llm_amd, m) {
   m.def("bm_talk_softmax(Tensor(a!) scores, Tensor pos, int H, float scale, Tensor? talk, bool act_f32) -> "
         "(Tensor, Tensor)");
   m.def("bm_moe_route(Tensor z, int top, int mode) -> (Tensor, Tensor)");
-  m.def("bm_moe_experts(Tensor h, Tensor idx, Tensor wts, Tensor w_gu, Tensor w_down, float limit, float alpha, "
-        "float up_shift, bool weigh_out) -> Tensor");
+  m.def("bm_moe_expert_rows(Tensor h, Tensor idx, Tensor wts, Tensor w_gu, Tensor w_down, float limit, float alpha, "
+        "float up_shift, bool weigh_out, int identity) -> Tensor");
 }
 
 TORCH_LIBRARY_IMPL(ipex_llm_amd, CompositeExplicitAutograd, m) {
@@ -456,5 +456,5 @@ TORCH_LIBRARY_IMPL(ipex_llm_amd, CUDA, m) {
   m.impl("bm_talk_prefill", &bm_talk_prefill);
   m.impl("bm_talk_softmax", &bm_talk_softmax);
   m.impl("bm_moe_route", &bm_moe_route);
-  m.impl("bm_moe_experts", &bm_moe_experts);
+  m.impl("bm_moe_expert_rows", &bm_moe_expert_rows);
 }

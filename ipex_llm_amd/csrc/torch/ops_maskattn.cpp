@@ -32,7 +32,7 @@ bool head_rows(const Tensor& t, at::ScalarType ty) {
 Tensor ma_qkv_norm_rope_store(const Tensor& q, const c10::optional<Tensor>& k, const c10::optional<Tensor>& v,
                               const c10::optional<Tensor>& qn, const c10::optional<Tensor>& kn, bool whole, double eps,
                               const c10::optional<Tensor>& table, int64_t layout, const Tensor& pos, const Tensor& slots,
-                              const c10::optional<Tensor>& rows) {
+                              const c10::optional<Tensor>& rows, const c10::optional<Tensor>& temp) {
   c10::DeviceGuard g(q.device());
   TORCH_CHECK(is_act(q) && head_rows(q, q.scalar_type()), "ma_qkv_norm_rope_store: q [T, H, d] (heads contiguous in a row)");
   const auto in_ty = q.scalar_type();
@@ -66,6 +66,8 @@ Tensor ma_qkv_norm_rope_store(const Tensor& q, const c10::optional<Tensor>& k, c
     dims = 2 * table->size(1);
     max_pos = table->size(0);
   }
+  TORCH_CHECK(!has(temp) || (temp->is_cuda() && temp->scalar_type() == at::kFloat && temp->is_contiguous() && temp->numel() == H),
+              "ma_qkv_norm_rope_store: temp f32 [H]");
   TORCH_CHECK(layout == 0 || layout == 1, "ma_qkv_norm_rope_store: layout 0 (pairs) or 1 (half)");
   TORCH_CHECK(H + G <= 8192, "ma_qkv_norm_rope_store: too many heads");
   check_idx(pos, at::kLong, T, "ma_qkv_norm_rope_store: pos int64 [T]");
@@ -76,8 +78,8 @@ Tensor ma_qkv_norm_rope_store(const Tensor& q, const c10::optional<Tensor>& k, c
                                 has(qn) ? qn->data_ptr() : nullptr, store && has(kn) ? kn->data_ptr() : nullptr, whole,
                                 (float)eps, has(table) ? table->data_ptr<float>() : nullptr, (int)max_pos, (int)dims,
                                 (int)layout, pos.data_ptr<int64_t>(), slots.data_ptr<int64_t>(),
-                                store ? rows->data_ptr() : nullptr, num_rows, qo.data_ptr<float>(), (int)T, (int)H, (int)G,
-                                (int)d, (int)dv, stream());
+                                store ? rows->data_ptr() : nullptr, num_rows, qo.data_ptr<float>(),
+                                has(temp) ? temp->data_ptr<float>() : nullptr, (int)T, (int)H, (int)G, (int)d, (int)dv, stream());
   return qo;
 }
 
@@ -194,9 +196,9 @@ Tensor ma_sigmoid_gate(Tensor& o, const Tensor& gate) {
   TORCH_CHECK(o.is_cuda() && o.dim() == 2 && is_act(o) && o.is_contiguous(), "ma_sigmoid_gate: o [T, C] contiguous");
   const int64_t T = o.size(0), C = o.size(1);
   TORCH_CHECK(gate.is_cuda() && gate.dim() == 2 && gate.scalar_type() == o.scalar_type() && gate.size(0) == T &&
-                  gate.size(1) == C && (C == 1 || gate.stride(1) == 1),
-              "ma_sigmoid_gate: gate [T, C] of o's dtype (unit inner stride)");
-  illm::ma::sigmoid_gate(bf(o), o.data_ptr(), gate.data_ptr(), gate.stride(0), T, (int)C, stream());
+                  gate.size(1) >= 1 && C % gate.size(1) == 0 && (gate.size(1) == 1 || gate.stride(1) == 1),
+              "ma_sigmoid_gate: gate [T, C] or [T, heads] of o's dtype (unit inner stride)");
+  illm::ma::sigmoid_gate(bf(o), o.data_ptr(), gate.data_ptr(), gate.stride(0), T, (int)C, (int)(C / gate.size(1)), stream());
   return o;
 }
 
@@ -204,7 +206,7 @@ Tensor ma_sigmoid_gate(Tensor& o, const Tensor& gate) {
 
 TORCH_LIBRARY_FRAGMENT(ipex_llm_amd, m) {
   m.def("ma_qkv_norm_rope_store(Tensor q, Tensor? k, Tensor? v, Tensor? qn, Tensor? kn, bool whole, float eps, "
-        "Tensor? table, int layout, Tensor pos, Tensor slots, Tensor(a!)? rows) -> Tensor");
+        "Tensor? table, int layout, Tensor pos, Tensor slots, Tensor(a!)? rows, Tensor? temp) -> Tensor");
   m.def("ma_masked_attention(Tensor q, Tensor rows, int G, int dv, Tensor block_tables, Tensor seq_of, Tensor pos, "
         "float scale, int mask, int size, Tensor? sink, int max_ctx, bool act_f32, float softcap, int keep_first, "
         "Tensor? talk) -> Tensor");
