@@ -186,7 +186,19 @@ def main():
     ap.add_argument("--twonorm-sizes", default="small,base")
     ap.add_argument("--twonorm-prompts", default="1024,4096")
     ap.add_argument("--no-twonorm-ref", action="store_true", help="--twonorm: skip the comparison model")
+    ap.add_argument("--sandwich", action="store_true",
+                    help="side benchmark (not the headline metric): prefill / decode throughput of the decoder normed "
+                         "before and after every sublayer (windowed attention beside a real-gated linear recurrent unit, "
+                         "gated delta rule, lightning attention, experts in groups) beside the decoder of two-norm "
+                         "parallel blocks at equal sizes, one GPU")
+    ap.add_argument("--sandwich-sizes", default="small,base")
+    ap.add_argument("--sandwich-prompts", default="1024,4096")
+    ap.add_argument("--no-sandwich-ref", action="store_true", help="--sandwich: skip the comparison model")
     args = ap.parse_args()
+    if args.sandwich:
+        from ipex_llm_amd.utils.bench_sandwich import main as sandwich_main
+        sandwich_main(args)
+        return
     if args.twonorm:
         from ipex_llm_amd.utils.bench_twonorm import main as twonorm_main
         twonorm_main(args)
