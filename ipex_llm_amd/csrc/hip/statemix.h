@@ -40,10 +40,30 @@ void decay_scan(bool bf16, const void* q, int64_t q_ld, const void* k, int64_t k
                 const float* decay, float* S, const int32_t* cu, const int32_t* slots, const int64_t* pos, float* out,
                 int B, int H, int d, int dv, hipStream_t st);
 // gated delta rule; q, k f32 rows [T, K d], v f32 [T, H dv]; a, b [T, H] in the activation type
+struct DeltaArgs {
+  const void* a;
+  int64_t a_ld;
+  const void* b;
+  int64_t b_ld;
+  const float* rate;
+  const float* dt_bias;
+  float q_scale, unit_eps;
+};
 void delta_scan(bool bf16, const float* q, int64_t q_ld, const float* k, int64_t k_ld, const float* v, int64_t v_ld,
-                const void* a, int64_t a_ld, const void* b, int64_t b_ld, const float* rate, const float* dt_bias,
-                float q_scale, float unit_eps, float* S, const int32_t* cu, const int32_t* slots, const int64_t* pos,
-                float* out, int B, int H, int K, int d, int dv, hipStream_t st);
+                DeltaArgs da, float* S, const int32_t* cu, const int32_t* slots, const int64_t* pos, float* out, int B, int H,
+                int K, int d, int dv, hipStream_t st);
+// the same two recurrences for long portions, in chunks of kChunk tokens on the matrix cores (statemix_chunk.hip): the
+// tokens [seg0, seg0 + seg) of every portion, nch chunks in all (a portion's last one may be short); the state is read
+// from and left in the slots.  Key sizes up to kChunkMaxDim
+constexpr int kChunk = 64;
+constexpr int kChunkMaxDim = 128;
+int64_t chunk_scratch_floats(bool delta, int64_t nch, int H, int d, int dv);
+void decay_chunks(bool bf16, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld,
+                  const float* decay, float* S, const int32_t* cu, const int32_t* slots, const int64_t* pos, float* out,
+                  float* scratch, int B, int nch, int seg0, int seg, int H, int d, int dv, hipStream_t st);
+void delta_chunks(bool bf16, const float* q, int64_t q_ld, const float* k, int64_t k_ld, const float* v, int64_t v_ld,
+                  DeltaArgs da, float* S, const int32_t* cu, const int32_t* slots, const int64_t* pos, float* out,
+                  float* scratch, int B, int nch, int seg0, int seg, int H, int K, int d, int dv, hipStream_t st);
 // block-diagonal gates: w_r, w_i [nb, n, n] in the activation type; u, a, x f32 [T, nb n]
 void rglru_gates(bool bf16, const float* u, const void* w_r, const float* b_r, const void* w_i, const float* b_i,
                  const float* log_base, float* a, float* x, int T, int nb, int n, hipStream_t st);

@@ -43,16 +43,6 @@ __device__ __forceinline__ float silu(float z) { return z / (1.0f + expf(-z)); }
 __device__ __forceinline__ float softplusf(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
 // ------------------------------------------------------------------ matrix-state scan, token by token
-struct DeltaArgs {
-  const void* a;
-  int64_t a_ld;
-  const void* b;
-  int64_t b_ld;
-  const float* rate;
-  const float* dt_bias;
-  float q_scale, unit_eps;
-};
-
 // EQ: type of q / k / v, EA: of the delta rule's a / b.  NC4: 16-row pieces of the state (d <= 16 NC4)
 template <typename EQ, typename EA, int NC4, bool DELTA>
 __global__ void __launch_bounds__(256) state_scan_k(const EQ* __restrict__ q, int64_t q_ld, const EQ* __restrict__ k,
@@ -406,10 +396,8 @@ void decay_scan(bool bf16, const void* q, int64_t q_ld, const void* k, int64_t k
 }
 
 void delta_scan(bool bf16, const float* q, int64_t q_ld, const float* k, int64_t k_ld, const float* v, int64_t v_ld,
-                const void* a, int64_t a_ld, const void* b, int64_t b_ld, const float* rate, const float* dt_bias,
-                float q_scale, float unit_eps, float* S, const int32_t* cu, const int32_t* slots, const int64_t* pos,
-                float* out, int B, int H, int K, int d, int dv, hipStream_t st) {
-  const DeltaArgs da{a, a_ld, b, b_ld, rate, dt_bias, q_scale, unit_eps};
+                DeltaArgs da, float* S, const int32_t* cu, const int32_t* slots, const int64_t* pos, float* out, int B, int H,
+                int K, int d, int dv, hipStream_t st) {
   if (bf16)
     launch_scan<float, __bf16, true>(q, q_ld, k, k_ld, v, v_ld, nullptr, da, S, cu, slots, pos, out, B, H, K, d, dv, st);
   else

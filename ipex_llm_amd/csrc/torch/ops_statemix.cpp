@@ -7,6 +7,7 @@
 #include <c10/core/DeviceGuard.h>
 #include <torch/library.h>
 
+#include <algorithm>
 #include <tuple>
 
 #include "../hip/statemix.h"
@@ -162,8 +163,37 @@ void check_state(const Tensor& S, int64_t H, int64_t d, int64_t dv, const char* 
               ": key size 1..", illm::sx::kScanMaxDim);
 }
 
+// portions of at least ``chunk_min`` tokens (0: never) run in chunks; long ones segment by segment, so that the scratch
+// memory stays bounded.  f(chunks, first token, tokens) launches one segment
+constexpr int64_t kSegment = 8192;
+bool by_chunks(c10::IntArrayRef lens, int64_t chunk_min, int64_t d) {
+  int64_t n = 0;
+  for (auto v : lens) n = std::max(n, v);
+  return chunk_min > 0 && n >= chunk_min && d <= illm::sx::kChunkMaxDim;
+}
+template <typename F> void segments(c10::IntArrayRef lens, F f) {
+  int64_t longest = 0;
+  for (auto v : lens) longest = std::max(longest, v);
+  for (int64_t s0 = 0; s0 < longest; s0 += kSegment) {
+    int64_t nch = 0;
+    for (auto v : lens) {
+      const int64_t n = std::min(kSegment, v - s0);
+      if (n > 0) nch += (n + illm::sx::kChunk - 1) / illm::sx::kChunk;
+    }
+    f((int)nch, (int)s0, (int)kSegment);
+  }
+}
+void check_lens(c10::IntArrayRef lens, const Tensor& cu, int64_t T, const char* what) {
+  int64_t sum = 0;
+  for (auto v : lens) {
+    TORCH_CHECK(v >= 0, what, ": negative portion");
+    sum += v;
+  }
+  TORCH_CHECK((int64_t)lens.size() == cu.numel() - 1 && sum == T, what, ": one length per sequence, T in all");
+}
+
 Tensor sx_decay_scan(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& decay, Tensor& S, const Tensor& cu,
-                     const Tensor& slots, const Tensor& pos) {
+                     const Tensor& slots, const Tensor& pos, c10::IntArrayRef lens, int64_t chunk_min) {
   c10::DeviceGuard g(q.device());
   const auto ty = q.scalar_type();
   TORCH_CHECK(is_act(q) && head_rows(q, ty) && head_rows(k, ty) && k.sizes() == q.sizes(),
@@ -176,6 +206,17 @@ Tensor sx_decay_scan(const Tensor& q, const Tensor& k, const Tensor& v, const Te
   check_step(cu, slots, pos, T, "sx_decay_scan");
   Tensor out = at::empty({T, H, dv}, q.options().dtype(at::kFloat));
   if (T == 0) return out;
+  check_lens(lens, cu, T, "sx_decay_scan");
+  if (by_chunks(lens, chunk_min, d)) {
+    segments(lens, [&](int nch, int s0, int seg) {
+      Tensor scratch = at::empty({illm::sx::chunk_scratch_floats(false, nch, (int)H, (int)d, (int)dv)}, out.options());
+      illm::sx::decay_chunks(bf(q), q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0),
+                             decay.data_ptr<float>(), S.data_ptr<float>(), cu.data_ptr<int32_t>(), slots.data_ptr<int32_t>(),
+                             pos.data_ptr<int64_t>(), out.data_ptr<float>(), scratch.data_ptr<float>(), (int)cu.numel() - 1,
+                             nch, s0, seg, (int)H, (int)d, (int)dv, stream());
+    });
+    return out;
+  }
   illm::sx::decay_scan(bf(q), q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0),
                        decay.data_ptr<float>(), S.data_ptr<float>(), cu.data_ptr<int32_t>(), slots.data_ptr<int32_t>(),
                        pos.data_ptr<int64_t>(), out.data_ptr<float>(), (int)cu.numel() - 1, (int)H, (int)d, (int)dv,
@@ -185,7 +226,7 @@ Tensor sx_decay_scan(const Tensor& q, const Tensor& k, const Tensor& v, const Te
 
 Tensor sx_delta_scan(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& a, const Tensor& b,
                      const Tensor& rate, const Tensor& dt_bias, double q_scale, double unit_eps, Tensor& S,
-                     const Tensor& cu, const Tensor& slots, const Tensor& pos) {
+                     const Tensor& cu, const Tensor& slots, const Tensor& pos, c10::IntArrayRef lens, int64_t chunk_min) {
   c10::DeviceGuard g(q.device());
   TORCH_CHECK(head_rows(q, at::kFloat) && head_rows(k, at::kFloat) && k.sizes() == q.sizes(),
               "sx_delta_scan: q, k f32 [T, K, d] (heads contiguous in a row)");
@@ -200,11 +241,23 @@ Tensor sx_delta_scan(const Tensor& q, const Tensor& k, const Tensor& v, const Te
   check_step(cu, slots, pos, T, "sx_delta_scan");
   Tensor out = at::empty({T, H, dv}, q.options());
   if (T == 0) return out;
+  check_lens(lens, cu, T, "sx_delta_scan");
+  const illm::sx::DeltaArgs da{a.data_ptr(), a.stride(0), b.data_ptr(), b.stride(0), rate.data_ptr<float>(),
+                               dt_bias.data_ptr<float>(), (float)q_scale, (float)unit_eps};
+  if (by_chunks(lens, chunk_min, d)) {
+    segments(lens, [&](int nch, int s0, int seg) {
+      Tensor scratch = at::empty({illm::sx::chunk_scratch_floats(true, nch, (int)H, (int)d, (int)dv)}, out.options());
+      illm::sx::delta_chunks(bf(a), q.data_ptr<float>(), q.stride(0), k.data_ptr<float>(), k.stride(0), v.data_ptr<float>(),
+                             v.stride(0), da, S.data_ptr<float>(), cu.data_ptr<int32_t>(), slots.data_ptr<int32_t>(),
+                             pos.data_ptr<int64_t>(), out.data_ptr<float>(), scratch.data_ptr<float>(), (int)cu.numel() - 1,
+                             nch, s0, seg, (int)H, (int)K, (int)d, (int)dv, stream());
+    });
+    return out;
+  }
   illm::sx::delta_scan(bf(a), q.data_ptr<float>(), q.stride(0), k.data_ptr<float>(), k.stride(0), v.data_ptr<float>(),
-                       v.stride(0), a.data_ptr(), a.stride(0), b.data_ptr(), b.stride(0), rate.data_ptr<float>(),
-                       dt_bias.data_ptr<float>(), (float)q_scale, (float)unit_eps, S.data_ptr<float>(),
-                       cu.data_ptr<int32_t>(), slots.data_ptr<int32_t>(), pos.data_ptr<int64_t>(), out.data_ptr<float>(),
-                       (int)cu.numel() - 1, (int)H, (int)K, (int)d, (int)dv, stream());
+                       v.stride(0), da, S.data_ptr<float>(), cu.data_ptr<int32_t>(), slots.data_ptr<int32_t>(),
+                       pos.data_ptr<int64_t>(), out.data_ptr<float>(), (int)cu.numel() - 1, (int)H, (int)K, (int)d, (int)dv,
+                       stream());
   return out;
 }
 
@@ -259,10 +312,10 @@ TORCH_LIBRARY_FRAGMENT(ipex_llm_amd, m) {
         "Tensor pw, Tensor pb, Tensor? qa, Tensor? qw, Tensor? qb, bool act_f32) -> Tensor");
   m.def("sx_rms_sigmoid_gate(Tensor o, Tensor w, Tensor gate, float eps, bool act_f32) -> Tensor");
   m.def("sx_route_groups(Tensor z, Tensor? corr, int top, int groups, int keep) -> (Tensor, Tensor)");
-  m.def("sx_decay_scan(Tensor q, Tensor k, Tensor v, Tensor decay, Tensor(a!) S, Tensor cu, Tensor slots, Tensor pos) "
-        "-> Tensor");
+  m.def("sx_decay_scan(Tensor q, Tensor k, Tensor v, Tensor decay, Tensor(a!) S, Tensor cu, Tensor slots, Tensor pos, "
+        "int[] lens, int chunk_min) -> Tensor");
   m.def("sx_delta_scan(Tensor q, Tensor k, Tensor v, Tensor a, Tensor b, Tensor rate, Tensor dt_bias, float q_scale, "
-        "float unit_eps, Tensor(a!) S, Tensor cu, Tensor slots, Tensor pos) -> Tensor");
+        "float unit_eps, Tensor(a!) S, Tensor cu, Tensor slots, Tensor pos, int[] lens, int chunk_min) -> Tensor");
   m.def("sx_rglru_gates(Tensor u, Tensor w_r, Tensor b_r, Tensor w_i, Tensor b_i, Tensor log_base) -> (Tensor, Tensor)");
   m.def("sx_rglru_scan(Tensor a, Tensor x, Tensor y, Tensor(a!) state, Tensor cu, Tensor slots, Tensor pos, int max_n) "
         "-> Tensor");

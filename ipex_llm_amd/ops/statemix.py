@@ -16,6 +16,7 @@ recurrences' sums are f32 whatever the activation dtype is.
 from __future__ import annotations
 
 import math
+import os
 from dataclasses import dataclass
 from typing import List, Optional, Tuple, Union
 
@@ -28,6 +29,10 @@ __all__ = ["PairMean", "ExpertSum", "dyn_tanh", "add_normed_", "decay_scan", "de
            "rglru_gates", "rglru_scan", "route_groups", "SCAN_MAX_DIM"]
 
 SCAN_MAX_DIM = 512             # largest key size per head the scan kernels hold (4 lanes x 128 state rows)
+
+# GPU: a step with a portion of at least CHUNK_MIN tokens (0: never) runs the matrix-state recurrences in chunks of 64
+# tokens on the matrix cores, other steps (decoding, short portions) token by token
+CHUNK_MIN = int(os.environ.get("ILLM_STATE_CHUNK_MIN", "64"))
 
 
 def _ops():
@@ -142,7 +147,7 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.T
     if native(q):
         if d > SCAN_MAX_DIM:
             raise ValueError(f"decay_scan: key size {d} is above the kernel's {SCAN_MAX_DIM}")
-        return _ops().sx_decay_scan(q, k, v, decay, state, cu, state_slots, pos)
+        return _ops().sx_decay_scan(q, k, v, decay, state, cu, state_slots, pos, q_lens, CHUNK_MIN)
     out = torch.empty(T, H, v.shape[2], dtype=torch.float32, device=q.device)
     qf, kf, vf = F.silu(q.float()), F.silu(k.float()), F.silu(v.float())
     dec = decay.float()[:, None, None]
@@ -179,7 +184,8 @@ def delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, a_pre: torch.T
     if native(q):
         if d > SCAN_MAX_DIM:
             raise ValueError(f"delta_scan: key size {d} is above the kernel's {SCAN_MAX_DIM}")
-        return _ops().sx_delta_scan(q, k, v, a_pre, b_pre, rate, dt_bias, q_scale, UNIT_EPS, state, cu, state_slots, pos)
+        return _ops().sx_delta_scan(q, k, v, a_pre, b_pre, rate, dt_bias, q_scale, UNIT_EPS, state, cu, state_slots,
+                                    pos, q_lens, CHUNK_MIN)
     rep = H // K
     out = torch.empty(T, H, dv, dtype=torch.float32, device=q.device)
 

@@ -186,10 +186,13 @@ def test_row_norm_with_sigmoid_gate(dev, act):
 SCAN_SIZES = [(3, 6, 10), (2, 48, 64), (1, 70, 70), (2, 130, 8), (1, 1, 1), (1, 300, 20), (4, 64, 128), (2, 16, 17)]
 
 
+@pytest.mark.parametrize("chunk_min", [0, 2])
 @pytest.mark.parametrize("H,d,dv", SCAN_SIZES)
-def test_decay_scan(dev, H, d, dv):
-    """a fixed decay per head (one near 1, one small); state carried over portions and batches, dirty slots"""
+def test_decay_scan(dev, H, d, dv, chunk_min, monkeypatch):
+    """a fixed decay per head (one near 1, one small); state carried over portions and batches, dirty slots; on the
+    GPU token by token and in chunks"""
     from ipex_llm_amd.ops import statemix as SX
+    monkeypatch.setattr(SX, "CHUNK_MIN", chunk_min)
     g = torch.Generator().manual_seed(H + d)
     decay = torch.tensor([0.999, 0.3, 0.9, 1.0][:H])
     for act in (torch.float32, torch.bfloat16):
@@ -225,11 +228,14 @@ def delta_want(q, k, v, ab, rate, bias, H):
     return O.delta_scan(O.unit(q) * q.shape[2] ** -0.5, O.unit(k), v, g, beta)
 
 
+@pytest.mark.parametrize("chunk_min", [0, 2])
 @pytest.mark.parametrize("H,K,d,dv", [(4, 2, 6, 10), (2, 2, 48, 64), (1, 1, 70, 70), (6, 2, 130, 8), (1, 1, 1, 1),
                                       (2, 1, 300, 20), (4, 4, 64, 128), (3, 1, 16, 17)])
-def test_delta_scan(dev, H, K, d, dv):
-    """the gated delta rule over portions and batches, key heads shared by several value heads, dirty slots"""
+def test_delta_scan(dev, H, K, d, dv, chunk_min, monkeypatch):
+    """the gated delta rule over portions and batches, key heads shared by several value heads, dirty slots; on the
+    GPU token by token and in chunks"""
     from ipex_llm_amd.ops import statemix as SX
+    monkeypatch.setattr(SX, "CHUNK_MIN", chunk_min)
     g = torch.Generator().manual_seed(H + d)
     rate, bias = torch.rand(H, generator=g), torch.randn(H, generator=g)
     for act in (torch.float32, torch.bfloat16):
@@ -249,6 +255,58 @@ def test_delta_scan(dev, H, K, d, dv):
         for i, o in zip(ins, in_portions(f, seqs, CUTS, dev)):
             want = delta_want(*i, rate, bias, H).reshape(o.shape)
             assert (o - want).abs().max() < 2e-5 * max(1.0, float(want.abs().max()))
+
+
+def test_long_portions_of_the_state_scans(dev):
+    """portions of thousands of tokens (on the GPU: many chunks, more than one segment of them) beside short ones and
+    one that continues; equal keys with steps near 1, and decays that all but clear the state now and then"""
+    from ipex_llm_amd.ops import statemix as SX
+    g = torch.Generator().manual_seed(6)
+    H, d, dv = 1, 5, 3
+    lens, starts = [8400, 1, 130, 64], [0, 9, 3, 0]
+    T = sum(lens)
+    cu, _, slots, pos = ragged(lens, starts, dev)
+    q, k, v = torch.randn(T, H, d, generator=g), torch.randn(T, H, d, generator=g), torch.randn(T, H, dv, generator=g)
+    k[100:300] = k[100]
+    a, b = torch.randn(T, H, generator=g) - 4, torch.randn(T, H, generator=g)
+    a[torch.arange(50, T, 97)] = 300.0
+    b[100:200] = 9.0
+    rate, bias, decay = torch.tensor([2.0]), torch.tensor([0.3]), torch.tensor([0.997])
+    S0 = torch.randn(6, H, d, dv, generator=g)
+
+    def check(got, state, step):
+        t0 = 0
+        for s, n in enumerate(lens):
+            S = torch.zeros(H, d, dv, dtype=F64) if starts[s] == 0 else S0[s + 1].double()
+            want = torch.empty(n, H, dv, dtype=F64)
+            for t in range(n):
+                S, want[t] = step(S, t0 + t)
+            tol = 3e-5 * max(1.0, float(want.abs().max()))
+            assert (got[t0:t0 + n].double().cpu() - want).abs().max() < tol, s
+            assert (state[s + 1].double().cpu() - S).abs().max() < 3e-5 * max(1.0, float(S.abs().max())), s
+            t0 += n
+
+    state = S0.clone().to(dev)
+    got = SX.decay_scan(q.to(dev), k.to(dev), v.to(dev), decay.to(dev), state, cu, slots, pos, lens)
+    qs, ks, vs = O.silu(q.double()), O.silu(k.double()), O.silu(v.double())
+
+    def light(S, t):
+        S = decay.double() * S + ks[t][:, :, None] * vs[t][:, None, :]
+        return S, (S * qs[t][:, :, None]).sum(1)
+    check(got, state, light)
+    state = S0.clone().to(dev)
+    got = SX.delta_scan(q.to(dev), k.to(dev), v.to(dev), a.to(dev), b.to(dev), rate.to(dev), bias.to(dev), 0.5, state, cu,
+                        slots, pos, lens)
+    qu, ku = O.unit(q.double()) * 0.5, O.unit(k.double())
+    gd = torch.exp(-2.0 * O.softplus(a.double() + bias.double()))
+    be = O.sigmoid(b.double())
+
+    def rule(S, t):
+        S = gd[t][:, None, None] * S
+        u = be[t][:, None] * (v[t].double() - (S * ku[t][:, :, None]).sum(1))
+        S = S + ku[t][:, :, None] * u[:, None, :]
+        return S, (S * qu[t][:, :, None]).sum(1)
+    check(got, state, rule)
 
 
 @pytest.mark.parametrize("nb,n", [(3, 8), (1, 5), (2, 35), (4, 64), (2, 136), (1, 1)])
