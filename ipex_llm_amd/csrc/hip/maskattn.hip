@@ -145,6 +145,79 @@ __global__ void __launch_bounds__(1024) qkv_store_k(const EI* __restrict__ q, in
     for (int e = threadIdx.x; e < G * dv; e += blockDim.x) stf(row + (int64_t)G * d + e, ldf(v + t * v_ld + e));
 }
 
+// the same step for per-head norms (or none) and neighbouring pairs: a wave per head, two neighbouring values per lane
+// held in registers (d even, at most 512), so every value is read once
+template <typename E> struct Two;
+template <> struct Two<float> {
+  static __device__ __forceinline__ void ld(const float* p, float* v) {
+    const float2 a = *(const float2*)p;
+    v[0] = a.x, v[1] = a.y;
+  }
+  static __device__ __forceinline__ void st(float* p, float a, float b) { *(float2*)p = make_float2(a, b); }
+};
+template <> struct Two<__bf16> {
+  typedef __bf16 B2 __attribute__((ext_vector_type(2)));
+  static __device__ __forceinline__ void ld(const __bf16* p, float* v) {
+    const B2 a = *(const B2*)p;
+    v[0] = (float)a[0], v[1] = (float)a[1];
+  }
+  static __device__ __forceinline__ void st(__bf16* p, float a, float b) { *(B2*)p = B2{(__bf16)a, (__bf16)b}; }
+};
+
+template <typename EI, typename E, int PL>
+__global__ void __launch_bounds__(1024) qkv_store_pairs_k(const EI* __restrict__ q, int64_t q_ld, const EI* __restrict__ k,
+                                                         int64_t k_ld, const EI* __restrict__ v, int64_t v_ld,
+                                                         const E* __restrict__ qn, const E* __restrict__ kn, float eps,
+                                                         const float* __restrict__ table, int dims,
+                                                         const int64_t* __restrict__ pos, const int64_t* __restrict__ slots,
+                                                         E* __restrict__ rows, float* __restrict__ qo,
+                                                         const float* __restrict__ temp, int H, int G, int d, int dv) {
+  const int64_t t = blockIdx.x;
+  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, NW = blockDim.x >> 6;
+  const int NK = H + (k ? G : 0), NA = NK + (k ? G : 0), half = d >> 1;
+  E* row = k ? rows + slots[t] * ((int64_t)G * (d + dv)) : nullptr;
+  const float* cs = table ? table + pos[t] * dims : nullptr;        // [dims / 2][2]
+  for (int hh = wv; hh < NA; hh += NW) {
+    if (hh >= NK) {                                                 // a value head
+      const EI* x = v + t * v_ld + (int64_t)(hh - NK) * dv;
+      E* o = row + (int64_t)G * d + (int64_t)(hh - NK) * dv;
+      for (int i = lane; i < dv; i += 64) stf(o + i, ldf(x + i));
+      continue;
+    }
+    const bool isq = hh < H;
+    const int head = isq ? hh : hh - H;
+    const EI* x = isq ? q + t * q_ld + (int64_t)head * d : k + t * k_ld + (int64_t)head * d;
+    const E* nw = isq ? qn : kn;
+    float a[PL][2];
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < PL; j++) {
+      const int i = lane + 64 * j;
+      a[j][0] = a[j][1] = 0.f;
+      if (i < half) Two<EI>::ld(x + 2 * i, a[j]);
+      ss = fmaf(a[j][0], a[j][0], fmaf(a[j][1], a[j][1], ss));
+    }
+    const float rs = nw ? 1.0f / sqrtf(wave_sum(ss) / (float)d + eps) : 1.0f;
+    const float tf = isq && temp ? temp[head] : 1.0f;
+#pragma unroll
+    for (int j = 0; j < PL; j++) {
+      const int i = lane + 64 * j;
+      if (i >= half) continue;
+      float w[2] = {1.f, 1.f};
+      if (nw) Two<E>::ld(nw + 2 * i, w);
+      float u0 = a[j][0] * rs * w[0], u1 = a[j][1] * rs * w[1];
+      if (cs && 2 * i < dims) {
+        const float2 r = *(const float2*)(cs + 2 * i);
+        const float n0 = u0 * r.x - u1 * r.y;
+        u1 = u1 * r.x + u0 * r.y;
+        u0 = n0;
+      }
+      if (isq) Two<float>::st(qo + (t * H + head) * d + 2 * i, u0 * tf, u1 * tf);
+      else Two<E>::st(row + (int64_t)head * d + 2 * i, u0, u1);
+    }
+  }
+}
+
 // ------------------------------------------------------------------ attention
 constexpr int KT = 16;                                              // keys per tile
 
@@ -512,14 +585,26 @@ __global__ void __launch_bounds__(256) chunk_softmax_k(float* __restrict__ sc, i
   }
 }
 
-// per: consecutive values that share a gate
-template <typename E>
+// per: consecutive values that share a gate.  V values per thread (V = 8: 16-byte accesses; C, and per unless it is 1,
+// are multiples of 8)
+template <typename E, int V>
 __global__ void __launch_bounds__(256) sigmoid_gate_k(E* __restrict__ o, const E* __restrict__ g, int64_t g_ld, int64_t n,
                                                      int C, int per) {
-  for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (int64_t)gridDim.x * blockDim.x) {
+  typedef E EV __attribute__((ext_vector_type(V)));
+  for (int64_t i = V * ((int64_t)blockIdx.x * blockDim.x + threadIdx.x); i < n; i += V * (int64_t)gridDim.x * blockDim.x) {
     const int64_t t = i / C;
     const int c = (int)(i - t * C);
-    stf(o + i, ldf(o + i) / (1.0f + expf(-ldf(g + t * g_ld + (per > 1 ? c / per : c)))));
+    EV x = *(const EV*)(o + i);
+    if (per > 1) {
+      const float f = 1.0f / (1.0f + expf(-ldf(g + t * g_ld + c / per)));
+#pragma unroll
+      for (int j = 0; j < V; j++) x[j] = (E)((float)x[j] * f);
+    } else {
+      const EV z = *(const EV*)(g + t * g_ld + c);
+#pragma unroll
+      for (int j = 0; j < V; j++) x[j] = (E)((float)x[j] / (1.0f + expf(-(float)z[j])));
+    }
+    *(EV*)(o + i) = x;
   }
 }
 
@@ -540,6 +625,27 @@ void qkv_norm_rope_store(bool in_bf16, bool bf16, const void* q, int64_t q_ld, c
   (void)max_pos;
   (void)num_rows;
   if (T <= 0) return;
+  const size_t ei = in_bf16 ? 2 : 4, eo = bf16 ? 2 : 4;
+  auto even = [](const void* p, size_t eb) { return (uintptr_t)p % (2 * eb) == 0; };
+  const bool row2 = ((int64_t)G * (d + dv)) % 2 == 0;               // a row starts at an even element
+  if (!whole && (!table || layout != kHalf) && d % 2 == 0 && d <= 512 && q_ld % 2 == 0 && even(q, ei) && even(qn, eo) &&
+      even(kn, eo) && (!k || (k_ld % 2 == 0 && even(k, ei) && even(rows, eo) && row2))) {
+    const int heads = H + (k ? 2 * G : 0), nw = T > 64 ? 4 : (heads < 16 ? heads : 16);
+#define MA_PAIRS(EI, E, PL)                                                                                             \
+  qkv_store_pairs_k<EI, E, PL><<<T, 64 * nw, 0, st>>>((const EI*)q, q_ld, (const EI*)k, k_ld, (const EI*)v, v_ld,       \
+                                                      (const E*)qn, (const E*)kn, eps, table, dims, pos, slots, (E*)rows, \
+                                                      qo, temp, H, G, d, dv)
+#define MA_PL(EI, E)                        \
+  if (d <= 128) MA_PAIRS(EI, E, 1);         \
+  else if (d <= 256) MA_PAIRS(EI, E, 2);    \
+  else MA_PAIRS(EI, E, 4)
+    if (bf16 && in_bf16) { MA_PL(__bf16, __bf16); }
+    else if (bf16) { MA_PL(float, __bf16); }
+    else { MA_PL(float, float); }
+#undef MA_PL
+#undef MA_PAIRS
+    return;
+  }
   const size_t lds = (size_t)(H + G + 2) * sizeof(float);
   // few tokens (decode): a thread per value or two, so that no thread walks a chain of dependent loads
   const int64_t vals = (int64_t)(H + G) * d;
@@ -651,9 +757,15 @@ void talk_mix(bool bf16, const float* w, const float* talk, int64_t pieces, int 
 void sigmoid_gate(bool bf16, void* o, const void* g, int64_t g_ld, int64_t T, int C, int per, hipStream_t st) {
   const int64_t n = T * C;
   if (n <= 0) return;
-  const int blocks = (int)((n + 255) / 256 > 65535 ? 65535 : (n + 255) / 256);
-  if (bf16) sigmoid_gate_k<__bf16><<<blocks, 256, 0, st>>>((__bf16*)o, (const __bf16*)g, g_ld, n, C, per);
-  else sigmoid_gate_k<float><<<blocks, 256, 0, st>>>((float*)o, (const float*)g, g_ld, n, C, per);
+  const size_t ab = 8 * (bf16 ? 2 : 4);
+  const bool v8 = C % 8 == 0 && (uintptr_t)o % ab == 0 &&
+                  (per > 1 ? per % 8 == 0 : (g_ld % 8 == 0 && (uintptr_t)g % ab == 0));
+  const int64_t nv = v8 ? n / 8 : n;
+  const int blocks = (int)((nv + 255) / 256 > 65535 ? 65535 : (nv + 255) / 256);
+#define MA_GATE(E, V) sigmoid_gate_k<E, V><<<blocks, 256, 0, st>>>((E*)o, (const E*)g, g_ld, n, C, per)
+  if (bf16) { if (v8) MA_GATE(__bf16, 8); else MA_GATE(__bf16, 1); }
+  else { if (v8) MA_GATE(float, 8); else MA_GATE(float, 1); }
+#undef MA_GATE
 }
 
 }  // namespace ma

@@ -32,6 +32,9 @@ void rms_sigmoid_gate(bool bf16, const float* o, const void* w, const void* gate
 // softmax over all E <= 512, choice by s + corr inside the best ``keep`` of ``groups`` groups, weights s
 void route_groups(const float* z, const float* corr, int T, int E, int top, int groups, int keep, int32_t* idx, float* w,
                   hipStream_t st);
+// the same from the router's input rows h [T, W] (activation type) and weights rw f32 [E, W]
+void router(bool bf16, const void* h, const float* rw, const float* corr, int T, int W, int E, int top, int groups,
+            int keep, int32_t* idx, float* w, hipStream_t st);
 
 // ---- recurrences (statemix_scan.hip)
 constexpr int kScanMaxDim = 512;

@@ -11,7 +11,8 @@
 //   RMS + sigmoid gate over the whole row
 //   group routing      one wave per token: softmax over all router outputs,
 //                      corrected scores and the groups' best ones in LDS, the
-//                      kept groups by rank, then the winners one after another
+//                      kept groups by rank, then the winners one after another;
+//                      for few tokens the same launch forms the logits
 //
 // Activations are bf16 or f32 (template E); all arithmetic is f32.
 #include "statemix.h"
@@ -205,19 +206,21 @@ __global__ void __launch_bounds__(1024) rms_sigmoid_gate_k(const float* __restri
 // ------------------------------------------------------------------ routing
 constexpr int kPerLane = 8;                                         // experts <= 512
 
-__global__ void __launch_bounds__(64) route_groups_k(const float* __restrict__ z, const float* __restrict__ corr, int E,
-                                                    int top, int groups, int keep, int32_t* __restrict__ idx,
-                                                    float* __restrict__ w) {
-  __shared__ float cs[64 * kPerLane];                               // corrected scores
-  __shared__ float best[64 * kPerLane];                             // per group; kept ones become 1, others 0
-  const int64_t t = blockIdx.x;
-  const int lane = threadIdx.x;
+// one wave routes token t with the logits z[0 .. E - 1]; cs, best: LDS of 64 kPerLane values
+__device__ __forceinline__ void wave_sync() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+__device__ void route_wave(const float* z, const float* __restrict__ corr, int E, int top, int groups, int keep,
+                           int32_t* __restrict__ idx, float* __restrict__ w, int64_t t, float* cs, float* best) {
+  const int lane = threadIdx.x & 63;
   float s[kPerLane], c[kPerLane];
   float mx = -INFINITY;
 #pragma unroll
   for (int i = 0; i < kPerLane; i++) {
     const int e = lane + 64 * i;
-    s[i] = e < E ? z[t * E + e] : -INFINITY;
+    s[i] = e < E ? z[e] : -INFINITY;
     mx = fmaxf(mx, s[i]);
   }
   mx = wave_max(mx);
@@ -237,13 +240,13 @@ __global__ void __launch_bounds__(64) route_groups_k(const float* __restrict__ z
   }
   if (keep < groups) {
     const int gs = E / groups;
-    __syncthreads();
+    wave_sync();
     for (int g = lane; g < groups; g += 64) {
       float b = -INFINITY;
       for (int j = 0; j < gs; j++) b = fmaxf(b, cs[g * gs + j]);
       best[g] = b;
     }
-    __syncthreads();
+    wave_sync();
     bool kept[kPerLane];
 #pragma unroll
     for (int i = 0; i < kPerLane; i++) {
@@ -255,11 +258,11 @@ __global__ void __launch_bounds__(64) route_groups_k(const float* __restrict__ z
       }
       kept[i] = g < groups && rank < keep;
     }
-    __syncthreads();
+    wave_sync();
 #pragma unroll
     for (int i = 0; i < kPerLane; i++)
       if (lane + 64 * i < groups) best[lane + 64 * i] = kept[i] ? 1.f : 0.f;
-    __syncthreads();
+    wave_sync();
 #pragma unroll
     for (int i = 0; i < kPerLane; i++) {
       const int e = lane + 64 * i;
@@ -297,6 +300,40 @@ __global__ void __launch_bounds__(64) route_groups_k(const float* __restrict__ z
         c[i] = -INFINITY;
       }
   }
+}
+
+__global__ void __launch_bounds__(64) route_groups_k(const float* __restrict__ z, const float* __restrict__ corr, int E,
+                                                    int top, int groups, int keep, int32_t* __restrict__ idx,
+                                                    float* __restrict__ w) {
+  __shared__ float cs[64 * kPerLane];                               // corrected scores
+  __shared__ float best[64 * kPerLane];                             // per group; kept ones become 1, others 0
+  const int64_t t = blockIdx.x;
+  route_wave(z + t * E, corr, E, top, groups, keep, idx, w, t, cs, best);
+}
+
+// few tokens: the logits as well (f32 products of the router with the token's row, a wave per router output), then the
+// first wave routes
+template <typename E, int V>
+__global__ void __launch_bounds__(1024) router_k(const E* __restrict__ h, const float* __restrict__ rw,
+                                                const float* __restrict__ corr, int W, int NE, int top, int groups, int keep,
+                                                int32_t* __restrict__ idx, float* __restrict__ w) {
+  __shared__ float cs[64 * kPerLane], best[64 * kPerLane], z[64 * kPerLane];
+  const int64_t t = blockIdx.x;
+  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, NW = blockDim.x >> 6;
+  for (int e = wv; e < NE; e += NW) {
+    float s = 0.f;
+    for (int c = V * lane; c < W; c += V * 64) {
+      float a[V], b[V];
+      Vec<E, V>::ld(h + t * W + c, a);
+      Vec<float, V>::ld(rw + (int64_t)e * W + c, b);
+#pragma unroll
+      for (int i = 0; i < V; i++) s = fmaf(a[i], b[i], s);
+    }
+    s = wave_sum(s);
+    if (lane == 0) z[e] = s;
+  }
+  __syncthreads();
+  if (wv == 0) route_wave(z, corr, NE, top, groups, keep, idx, w, t, cs, best);
 }
 
 int row_threads(int W, int V) {
@@ -364,6 +401,15 @@ void route_groups(const float* z, const float* corr, int T, int E, int top, int 
                   hipStream_t st) {
   if (T <= 0) return;
   route_groups_k<<<T, 64, 0, st>>>(z, corr, E, top, groups, keep, idx, w);
+}
+
+void router(bool bf16, const void* h, const float* rw, const float* corr, int T, int W, int E, int top, int groups,
+            int keep, int32_t* idx, float* w, hipStream_t st) {
+  if (T <= 0) return;
+  const int nt = 64 * (E < 16 ? E : 16);
+#define CALL(EL, V) (router_k<EL, V><<<T, nt, 0, st>>>((const EL*)h, rw, corr, W, E, top, groups, keep, idx, w))
+  if (bf16) { SX_V(W, CALL(__bf16, 1), CALL(__bf16, 4)) } else { SX_V(W, CALL(float, 1), CALL(float, 4)) }
+#undef CALL
 }
 
 }  // namespace sx

@@ -14,8 +14,9 @@
 //                      weights the f32 inputs are split into three 16-bit parts
 //                      (hi + mid + lo is the f32 number), so the sums carry f32
 //                      precision
-//   LRU scan           S' = a S + x per channel: pieces of a portion folded side
-//                      by side, their carries chained in order, then run again
+//   LRU scan           S' = a S + x per channel: up to 64 pieces of a portion
+//                      folded side by side, their carries chained in order, then
+//                      run again
 //
 // Activations are bf16 or f32 (template E); accumulation is always f32.
 #include "statemix.h"
@@ -254,6 +255,12 @@ __global__ void __launch_bounds__(256) rglru_gates_k(const float* __restrict__ u
 #pragma unroll
   for (int m = 0; m < MS; m++) ar[m] = ai[m] = f32x4{0.f, 0.f, 0.f, 0.f};
   for (int k0 = 0; k0 < n; k0 += KC) {
+    Frag<E> br[KC / 32], bi[KC / 32];                               // requested before the tokens' values are staged
+#pragma unroll
+    for (int ks = 0; ks < KC / 32; ks++) {
+      br[ks].load(wr, k0 + 32 * ks + 8 * g, ok ? n : 0, vec);
+      bi[ks].load(wi, k0 + 32 * ks + 8 * g, ok ? n : 0, vec);
+    }
     __syncthreads();
     for (int i = tid; i < TM * KC; i += 256) {
       const int r = i / KC, c = i - r * KC;
@@ -272,10 +279,6 @@ __global__ void __launch_bounds__(256) rglru_gates_k(const float* __restrict__ u
     __syncthreads();
 #pragma unroll
     for (int ks = 0; ks < KC / 32; ks++) {
-      const int kk = k0 + 32 * ks + 8 * g;
-      Frag<E> br, bi;
-      br.load(wr, kk, ok ? n : 0, vec);
-      bi.load(wi, kk, ok ? n : 0, vec);
 #pragma unroll
       for (int m = 0; m < MS; m++) {
 #pragma unroll
@@ -283,13 +286,13 @@ __global__ void __launch_bounds__(256) rglru_gates_k(const float* __restrict__ u
           const E* up = us[p] + (m * 16 + r16) * LP + 32 * ks + 8 * g;
           if constexpr (sizeof(E) == 2) {
             const bf16x8 a = *(const bf16x8*)up;
-            ar[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, br.v8(), ar[m], 0, 0, 0);
-            ai[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, bi.v8(), ai[m], 0, 0, 0);
+            ar[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, br[ks].v8(), ar[m], 0, 0, 0);
+            ai[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, bi[ks].v8(), ai[m], 0, 0, 0);
           } else {
 #pragma unroll
             for (int j = 0; j < 8; j++) {
-              ar[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(up[j], br.v[j], ar[m], 0, 0, 0);
-              ai[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(up[j], bi.v[j], ai[m], 0, 0, 0);
+              ar[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(up[j], br[ks].v[j], ar[m], 0, 0, 0);
+              ai[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(up[j], bi[ks].v[j], ai[m], 0, 0, 0);
             }
           }
         }
@@ -316,17 +319,17 @@ __device__ __forceinline__ float gelu_tanh(float z) {
   return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
 
-// thread (lane = channel, wave = piece); LDS: factors [16][64], results [16][64]
-template <typename E>
+// a workgroup: CW channels x NC pieces of a portion, thread = (piece, channel).  CW = 16 for long portions (more pieces,
+// more workgroups), 64 for decoded tokens
+template <typename E, int CW>
 __global__ void __launch_bounds__(1024) rglru_scan_k(const float* __restrict__ a, const float* __restrict__ x,
                                                     const E* __restrict__ y, int64_t y_ld, float* __restrict__ state,
                                                     const int32_t* __restrict__ cu, const int32_t* __restrict__ slots,
                                                     const int64_t* __restrict__ pos, E* __restrict__ out, int C) {
-  __shared__ float fa[16][64];
-  __shared__ float fb[16][64];
+  __shared__ float fa[1024], fb[1024];                              // the pieces' factors and results, [NC][CW]
   const int b = blockIdx.y;
-  const int lane = threadIdx.x & 63, j = threadIdx.x >> 6, NC = blockDim.x >> 6;
-  const int c = blockIdx.x * 64 + lane;
+  const int ch = threadIdx.x % CW, j = threadIdx.x / CW, NC = blockDim.x / CW;
+  const int c = blockIdx.x * CW + ch;
   const int t0 = cu[b], n = cu[b + 1] - t0;
   if (n <= 0) return;
   const bool ok = c < C;
@@ -352,13 +355,13 @@ __global__ void __launch_bounds__(1024) rglru_scan_k(const float* __restrict__ a
           Bv = fmaf(av[i], Bv, xv[i]);
         }
       }
-    fa[j][lane] = A;
-    fb[j][lane] = Bv;
+    fa[threadIdx.x] = A;
+    fb[threadIdx.x] = Bv;
     __syncthreads();
   }
   float* st = state + (int64_t)slots[b] * C + (ok ? c : 0);
   float S = (ok && pos[t0] != 0) ? *st : 0.f;
-  for (int jj = 0; jj < j; jj++) S = fmaf(fa[jj][lane], S, fb[jj][lane]);    // the carries in order
+  for (int jj = 0; jj < j; jj++) S = fmaf(fa[jj * CW + ch], S, fb[jj * CW + ch]);    // the carries in order
   __syncthreads();                                                  // every piece has read the slot
   if (!ok) return;
   const E* yp = y + (int64_t)t0 * y_ld + c;
@@ -422,13 +425,18 @@ void rglru_gates(bool bf16, const float* u, const void* w_r, const float* b_r, c
 void rglru_scan(bool bf16, const float* a, const float* x, const void* y, int64_t y_ld, float* state, const int32_t* cu,
                 const int32_t* slots, const int64_t* pos, void* out, int B, int C, int max_n, hipStream_t st) {
   if (B <= 0 || C <= 0) return;
-  // pieces per portion: at least 16 tokens a piece, as many as fill the chip, at most 16
-  const int64_t groups = (int64_t)B * ((C + 63) / 64);
+  // pieces per portion: at least 16 tokens a piece, at most 64 of them
   int nc = 1;
-  while (nc < 16 && max_n >= 32 * nc && groups * nc < 1024) nc *= 2;
-  const dim3 grid((C + 63) / 64, B), block(64 * nc);
-  if (bf16) rglru_scan_k<__bf16><<<grid, block, 0, st>>>(a, x, (const __bf16*)y, y_ld, state, cu, slots, pos, (__bf16*)out, C);
-  else rglru_scan_k<float><<<grid, block, 0, st>>>(a, x, (const float*)y, y_ld, state, cu, slots, pos, (float*)out, C);
+  while (nc < 64 && max_n >= 32 * nc) nc *= 2;
+#define SX_LRU(E, CW)                                                                                                  \
+  rglru_scan_k<E, CW><<<dim3((C + CW - 1) / CW, B), CW * nc, 0, st>>>(a, x, (const E*)y, y_ld, state, cu, slots, pos, \
+                                                                      (E*)out, C)
+  if (nc >= 4) {
+    if (bf16) SX_LRU(__bf16, 16); else SX_LRU(float, 16);
+  } else {
+    if (bf16) SX_LRU(__bf16, 64); else SX_LRU(float, 64);
+  }
+#undef SX_LRU
 }
 
 }  // namespace sx

@@ -155,6 +155,23 @@ std::tuple<Tensor, Tensor> sx_route_groups(const Tensor& z, const OptT& corr, in
   return {idx, w};
 }
 
+std::tuple<Tensor, Tensor> sx_router(const Tensor& h, const Tensor& rw, const OptT& corr, int64_t top, int64_t groups,
+                                     int64_t keep) {
+  c10::DeviceGuard g(h.device());
+  TORCH_CHECK(h.is_cuda() && h.dim() == 2 && is_act(h) && h.is_contiguous(), "sx_router: h [T, W] contiguous");
+  const int64_t T = h.size(0), W = h.size(1), E = rw.dim() == 2 ? rw.size(0) : 0;
+  TORCH_CHECK(rows(rw, at::kFloat, E, W), "sx_router: router f32 [E, W]");
+  TORCH_CHECK(E >= 1 && E <= 512 && groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && top >= 1 &&
+                  top <= keep * (E / groups),
+              "sx_router: E <= 512, equal groups, 1 <= top <= outputs of the kept groups");
+  TORCH_CHECK(!has(corr) || vec(*corr, at::kFloat, E), "sx_router: correction f32 [E]");
+  auto f = h.options().dtype(at::kFloat);
+  Tensor idx = at::empty({T, top}, f.dtype(at::kInt)), w = at::empty({T, top}, f);
+  illm::sx::router(bf(h), h.data_ptr(), rw.data_ptr<float>(), has(corr) ? corr->data_ptr<float>() : nullptr, (int)T, (int)W,
+                   (int)E, (int)top, (int)groups, (int)keep, idx.data_ptr<int32_t>(), w.data_ptr<float>(), stream());
+  return {idx, w};
+}
+
 void check_state(const Tensor& S, int64_t H, int64_t d, int64_t dv, const char* what) {
   TORCH_CHECK(S.is_cuda() && S.scalar_type() == at::kFloat && S.is_contiguous() && S.dim() == 4 && S.size(1) == H &&
                   S.size(2) == d && S.size(3) == dv,
@@ -312,6 +329,7 @@ TORCH_LIBRARY_FRAGMENT(ipex_llm_amd, m) {
         "Tensor pw, Tensor pb, Tensor? qa, Tensor? qw, Tensor? qb, bool act_f32) -> Tensor");
   m.def("sx_rms_sigmoid_gate(Tensor o, Tensor w, Tensor gate, float eps, bool act_f32) -> Tensor");
   m.def("sx_route_groups(Tensor z, Tensor? corr, int top, int groups, int keep) -> (Tensor, Tensor)");
+  m.def("sx_router(Tensor h, Tensor rw, Tensor? corr, int top, int groups, int keep) -> (Tensor, Tensor)");
   m.def("sx_decay_scan(Tensor q, Tensor k, Tensor v, Tensor decay, Tensor(a!) S, Tensor cu, Tensor slots, Tensor pos, "
         "int[] lens, int chunk_min) -> Tensor");
   m.def("sx_delta_scan(Tensor q, Tensor k, Tensor v, Tensor a, Tensor b, Tensor rate, Tensor dt_bias, float q_scale, "
@@ -328,6 +346,7 @@ TORCH_LIBRARY_IMPL(ipex_llm_amd, CUDA, m) {
   m.impl("sx_add_normed_experts", &sx_add_normed_experts);
   m.impl("sx_rms_sigmoid_gate", &sx_rms_sigmoid_gate);
   m.impl("sx_route_groups", &sx_route_groups);
+  m.impl("sx_router", &sx_router);
   m.impl("sx_decay_scan", &sx_decay_scan);
   m.impl("sx_delta_scan", &sx_delta_scan);
   m.impl("sx_rglru_gates", &sx_rglru_gates);

@@ -932,7 +932,7 @@ class ScoredMoE(nn.Module):
     def parts(self, xa) -> SX.ExpertSum:
         """the chosen experts' weighted results, their sum still to be formed"""
         s = self.s
-        idx, wts = SX.route_groups(F.linear(xa.float(), self.router), self.correction, s.top, s.groups, s.keep)
+        idx, wts = SX.route(xa, self.router, self.correction, s.top, s.groups, s.keep)
         rows = BM.moe_expert_rows(xa, idx, wts, self.w_gu, self.w_down, float("inf"), 1.0, 0.0, "output", s.identity)
         return SX.ExpertSum(rows, idx, wts, xa, s.experts)
 

@@ -26,7 +26,7 @@ import torch.nn.functional as F
 from .seqmix import native
 
 __all__ = ["PairMean", "ExpertSum", "dyn_tanh", "add_normed_", "decay_scan", "delta_scan", "rms_sigmoid_gate",
-           "rglru_gates", "rglru_scan", "route_groups", "SCAN_MAX_DIM"]
+           "rglru_gates", "rglru_scan", "route_groups", "route", "SCAN_MAX_DIM"]
 
 SCAN_MAX_DIM = 512             # largest key size per head the scan kernels hold (4 lanes x 128 state rows)
 
@@ -273,3 +273,15 @@ def route_groups(z: torch.Tensor, correction: Optional[torch.Tensor], top: int, 
         c = c.masked_fill(~ok.repeat_interleave(E // groups, 1), float("-inf"))
     idx = torch.sort(c, dim=-1, descending=True, stable=True).indices[:, :top]
     return idx.to(torch.int32).contiguous(), s.gather(1, idx).contiguous()
+
+
+ROUTER_MAX_T = 64              # GPU: up to this many tokens the logits and the routing are one launch
+
+
+def route(h: torch.Tensor, router: torch.Tensor, correction: Optional[torch.Tensor], top: int, groups: int,
+          keep: int) -> Tuple[torch.Tensor, torch.Tensor]:
+    """``route_groups`` of the logits ``h router^T`` (f32 products; ``h`` [T, W] in the activation dtype, ``router``
+    f32 [E, W])"""
+    if native(h) and h.shape[0] <= ROUTER_MAX_T and router.shape[0] <= 512:
+        return _ops().sx_router(h.contiguous(), router, correction, top, groups, keep)
+    return route_groups(F.linear(h.float(), router), correction, top, groups, keep)

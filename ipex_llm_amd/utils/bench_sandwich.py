@@ -50,7 +50,7 @@ def sandwich_config(sz: dict) -> dict:
     return {"architecture": "Sudosun", "vocab": sz["vocab"], "width": sz["width"], "norm": {"eps": 1e-6}, "logit_scale": 1.0,
             "layers": [{"type": "parallel", "mixer": pair, "mlp": moe}, {"type": "delta", "mixer": delta, "mlp": moe},
                        {"type": "lightning", "mixer": lightning, "mlp": dense},
-                       {"type": "parallel", "mixer": pair, "mlp": dense}]}
+                       {"type": "parallel", "mixer": pair, "mlp": moe}]}
 
 
 def reference_config(sz: dict) -> dict:

@@ -379,6 +379,22 @@ def test_routing_in_groups(dev, E, top, groups, keep):
             assert (w[t].double().cpu() - torch.stack([s for _, s in want])).abs().max() < 1e-6
 
 
+@pytest.mark.parametrize("act", [torch.float32, torch.bfloat16])
+def test_router_logits_and_choice(dev, act):
+    """few tokens (on the GPU one launch) and many (a product, then the choice)"""
+    from ipex_llm_amd.ops import statemix as SX
+    g = torch.Generator().manual_seed(9)
+    for T, Wd, E, top, groups, keep in ((3, 37, 6, 2, 3, 2), (64, 40, 20, 4, 4, 3), (65, 40, 20, 4, 4, 3), (1, 300, 33, 1, 1, 1)):
+        h = torch.randn(T, Wd, generator=g).to(act)
+        rw, corr = torch.randn(E, Wd, generator=g), 0.1 * torch.randn(E, generator=g)
+        idx, w = SX.route(h.to(dev), rw.to(dev), corr.to(dev), top, groups, keep)
+        z = h.double() @ rw.double().T
+        for t in range(T):
+            want = O.route(z[t], corr.double(), top, {"count": groups, "keep": keep})
+            assert idx[t].tolist() == [e for e, _ in want]
+            assert (w[t].double().cpu() - torch.stack([s for _, s in want])).abs().max() < 1e-5
+
+
 def test_group_choice_shows(dev):
     """two groups: the best score decides the group, the second best score of all sits in the other group and loses"""
     from ipex_llm_amd.ops import statemix as SX
