@@ -322,6 +322,7 @@ __global__ void __launch_bounds__(1024) router_k(const E* __restrict__ h, const 
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, NW = blockDim.x >> 6;
   for (int e = wv; e < NE; e += NW) {
     float s = 0.f;
+#pragma unroll 4
     for (int c = V * lane; c < W; c += V * 64) {
       float a[V], b[V];
       Vec<E, V>::ld(h + t * W + c, a);

@@ -233,6 +233,17 @@ template <typename E> struct Frag {
   __device__ __forceinline__ bf16x8 v8() const { return *(const bf16x8*)v; }
 };
 
+// an f32 value as the parts of E whose sum it is
+template <int N> __device__ __forceinline__ void stage(float (*us)[N], int at, float v) { us[0][at] = v; }
+template <int N> __device__ __forceinline__ void stage(__bf16 (*us)[N], int at, float v) {
+  const __bf16 hi = (__bf16)v;
+  const float r1 = v - (float)hi;
+  const __bf16 mid = (__bf16)r1;
+  us[0][at] = hi;
+  us[1][at] = mid;
+  us[2][at] = (__bf16)(r1 - (float)mid);
+}
+
 template <typename E, int TM>
 __global__ void __launch_bounds__(256) rglru_gates_k(const float* __restrict__ u, const E* __restrict__ w_r,
                                                     const float* __restrict__ b_r, const E* __restrict__ w_i,
@@ -262,18 +273,21 @@ __global__ void __launch_bounds__(256) rglru_gates_k(const float* __restrict__ u
       bi[ks].load(wi, k0 + 32 * ks + 8 * g, ok ? n : 0, vec);
     }
     __syncthreads();
-    for (int i = tid; i < TM * KC; i += 256) {
-      const int r = i / KC, c = i - r * KC;
-      const float v = (t0 + r < T && k0 + c < n) ? u[(int64_t)(t0 + r) * C + (int64_t)blk * n + k0 + c] : 0.f;
-      if constexpr (NP == 1) {
-        us[0][r * LP + c] = v;
-      } else {
-        const E hi = (E)v;
-        const float r1 = v - (float)hi;
-        const E mid = (E)r1;
-        us[0][r * LP + c] = hi;
-        us[1][r * LP + c] = mid;
-        us[2][r * LP + c] = (E)(r1 - (float)mid);
+    if (vec) {                                                      // rows are 16-byte aligned: four values at a time
+      for (int i = tid; i < TM * KC / 4; i += 256) {
+        const int r = i / (KC / 4), c = 4 * (i - r * (KC / 4));
+        float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (t0 + r < T && k0 + c < n) v = *(const float4*)(u + (int64_t)(t0 + r) * C + (int64_t)blk * n + k0 + c);
+        stage(us, r * LP + c, v.x);
+        stage(us, r * LP + c + 1, v.y);
+        stage(us, r * LP + c + 2, v.z);
+        stage(us, r * LP + c + 3, v.w);
+      }
+    } else {
+      for (int i = tid; i < TM * KC; i += 256) {
+        const int r = i / KC, c = i - r * KC;
+        stage(us, r * LP + c,
+              (t0 + r < T && k0 + c < n) ? u[(int64_t)(t0 + r) * C + (int64_t)blk * n + k0 + c] : 0.f);
       }
     }
     __syncthreads();

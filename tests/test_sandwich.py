@@ -727,6 +727,24 @@ def test_long_windows_take_the_product_path(dev, window, sizes, monkeypatch):
         assert rel_err(got, want) < TOL[dtype]
 
 
+def test_mixed_steps_at_matrix_core_sizes(dev):
+    """sizes that fill matrix-core tiles and ones that do not, long portions beside decoded tokens, both number formats"""
+    cfg = O.config([O.pair_layer(heads=4, kv_heads=2, dim=40, vdim=56, window=50, dims=20, width=144, blocks=3, taps=4,
+                                 mlp=O.moe(8, 4, 4, 40, (4, 3))),
+                    O.delta_layer(heads=4, kv_heads=2, dim=80, vdim=48, taps=4, mlp=O.dense_ff(96, 1.5)),
+                    O.lightning_layer(heads=2, dim=100, vdim=36, decay=[0.99, 0.7], mlp=O.moe(6, 2, 2, 64, (2, 1)))],
+                   vocab=120, width=96)
+    W = O.random_weights(cfg, 18)
+    P = {"a": O.random_tokens(cfg, 260, 1), "b": O.random_tokens(cfg, 90, 2), "c": O.random_tokens(cfg, 150, 3)}
+    schedule = [[("a", 100), ("b", 1)], [("a", 1), ("b", 2), ("c", 130)], [("a", 65), ("b", 86)],
+                [("a", 92), ("b", 1), ("c", 19)], [("a", 1)], [("a", 1), ("c", 1)]]
+    for dtype in (torch.float32, torch.bfloat16):
+        got = replay(engine(cfg, W, dev, dtype), P, schedule)
+        for name, toks in P.items():
+            # 16-bit: the worst of hundreds of rows, a router's close calls among them
+            assert rel_err(got[name], oracle(cfg, W, toks, "m18" + name)) < (TOL[dtype] if dtype == torch.float32 else 0.3), name
+
+
 def test_greedy_generation_scheduler(dev):
     """LLMEngine.generate: C++ scheduler, chunked prompts (7 tokens a step in all), requests of unequal
     length side by side, greedy sampling"""
