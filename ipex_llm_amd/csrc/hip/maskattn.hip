@@ -145,77 +145,96 @@ __global__ void __launch_bounds__(1024) qkv_store_k(const EI* __restrict__ q, in
     for (int e = threadIdx.x; e < G * dv; e += blockDim.x) stf(row + (int64_t)G * d + e, ldf(v + t * v_ld + e));
 }
 
-// the same step for per-head norms (or none) and neighbouring pairs: a wave per head, two neighbouring values per lane
-// held in registers (d even, at most 512), so every value is read once
-template <typename E> struct Two;
-template <> struct Two<float> {
-  static __device__ __forceinline__ void ld(const float* p, float* v) {
-    const float2 a = *(const float2*)p;
-    v[0] = a.x, v[1] = a.y;
+// the same step for per-head norms (or none) and neighbouring pairs: eight neighbouring values per lane, LPH lanes per
+// head (a power of two), 64 / LPH heads per wave, every value read once (d and dv multiples of 8, d <= 8 LPH)
+template <typename E> struct Eight {
+  typedef E V8 __attribute__((ext_vector_type(8)));
+  static __device__ __forceinline__ void ld(const E* p, float* v) {
+    const V8 a = *(const V8*)p;
+#pragma unroll
+    for (int i = 0; i < 8; i++) v[i] = (float)a[i];
   }
-  static __device__ __forceinline__ void st(float* p, float a, float b) { *(float2*)p = make_float2(a, b); }
-};
-template <> struct Two<__bf16> {
-  typedef __bf16 B2 __attribute__((ext_vector_type(2)));
-  static __device__ __forceinline__ void ld(const __bf16* p, float* v) {
-    const B2 a = *(const B2*)p;
-    v[0] = (float)a[0], v[1] = (float)a[1];
+  static __device__ __forceinline__ void st(E* p, const float* v) {
+    V8 a;
+#pragma unroll
+    for (int i = 0; i < 8; i++) a[i] = (E)v[i];
+    *(V8*)p = a;
   }
-  static __device__ __forceinline__ void st(__bf16* p, float a, float b) { *(B2*)p = B2{(__bf16)a, (__bf16)b}; }
 };
 
-template <typename EI, typename E, int PL>
-__global__ void __launch_bounds__(1024) qkv_store_pairs_k(const EI* __restrict__ q, int64_t q_ld, const EI* __restrict__ k,
-                                                         int64_t k_ld, const EI* __restrict__ v, int64_t v_ld,
-                                                         const E* __restrict__ qn, const E* __restrict__ kn, float eps,
-                                                         const float* __restrict__ table, int dims,
-                                                         const int64_t* __restrict__ pos, const int64_t* __restrict__ slots,
-                                                         E* __restrict__ rows, float* __restrict__ qo,
-                                                         const float* __restrict__ temp, int H, int G, int d, int dv) {
+template <typename EI, typename E, int LPH>
+__global__ void __launch_bounds__(512) qkv_store_pairs_k(const EI* __restrict__ q, int64_t q_ld, const EI* __restrict__ k,
+                                                        int64_t k_ld, const EI* __restrict__ v, int64_t v_ld,
+                                                        const E* __restrict__ qn, const E* __restrict__ kn, float eps,
+                                                        const float* __restrict__ table, int dims,
+                                                        const int64_t* __restrict__ pos, const int64_t* __restrict__ slots,
+                                                        E* __restrict__ rows, float* __restrict__ qo,
+                                                        const float* __restrict__ temp, int H, int G, int d, int dv) {
   const int64_t t = blockIdx.x;
-  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, NW = blockDim.x >> 6;
-  const int NK = H + (k ? G : 0), NA = NK + (k ? G : 0), half = d >> 1;
+  const int ln = threadIdx.x & (LPH - 1), i0 = 8 * ln;
+  const int NK = H + (k ? G : 0), per = blockDim.x / LPH;           // heads per pass
   E* row = k ? rows + slots[t] * ((int64_t)G * (d + dv)) : nullptr;
-  const float* cs = table ? table + pos[t] * dims : nullptr;        // [dims / 2][2]
-  for (int hh = wv; hh < NA; hh += NW) {
-    if (hh >= NK) {                                                 // a value head
-      const EI* x = v + t * v_ld + (int64_t)(hh - NK) * dv;
-      E* o = row + (int64_t)G * d + (int64_t)(hh - NK) * dv;
-      for (int i = lane; i < dv; i += 64) stf(o + i, ldf(x + i));
-      continue;
-    }
-    const bool isq = hh < H;
-    const int head = isq ? hh : hh - H;
-    const EI* x = isq ? q + t * q_ld + (int64_t)head * d : k + t * k_ld + (int64_t)head * d;
-    const E* nw = isq ? qn : kn;
-    float a[PL][2];
-    float ss = 0.f;
+  float cs[8];                                                      // this lane's four pairs: (cos, sin)
+  const bool turn = table && i0 < dims;
+  if (turn) {
+    const float* p = table + pos[t] * dims + i0;
 #pragma unroll
-    for (int j = 0; j < PL; j++) {
-      const int i = lane + 64 * j;
-      a[j][0] = a[j][1] = 0.f;
-      if (i < half) Two<EI>::ld(x + 2 * i, a[j]);
-      ss = fmaf(a[j][0], a[j][0], fmaf(a[j][1], a[j][1], ss));
-    }
-    const float rs = nw ? 1.0f / sqrtf(wave_sum(ss) / (float)d + eps) : 1.0f;
-    const float tf = isq && temp ? temp[head] : 1.0f;
-#pragma unroll
-    for (int j = 0; j < PL; j++) {
-      const int i = lane + 64 * j;
-      if (i >= half) continue;
-      float w[2] = {1.f, 1.f};
-      if (nw) Two<E>::ld(nw + 2 * i, w);
-      float u0 = a[j][0] * rs * w[0], u1 = a[j][1] * rs * w[1];
-      if (cs && 2 * i < dims) {
-        const float2 r = *(const float2*)(cs + 2 * i);
-        const float n0 = u0 * r.x - u1 * r.y;
-        u1 = u1 * r.x + u0 * r.y;
-        u0 = n0;
-      }
-      if (isq) Two<float>::st(qo + (t * H + head) * d + 2 * i, u0 * tf, u1 * tf);
-      else Two<E>::st(row + (int64_t)head * d + 2 * i, u0, u1);
+    for (int i = 0; i < 8; i += 2) {
+      const float2 r = i0 + i < dims ? *(const float2*)(p + i) : make_float2(1.f, 0.f);
+      cs[i] = r.x;
+      cs[i + 1] = r.y;
     }
   }
+  const bool in = i0 < d;
+  const bool normed = qn || kn;
+  for (int h0 = 0; h0 < NK; h0 += per) {
+    const int hh = h0 + threadIdx.x / LPH;
+    const bool isq = hh < H, ok = in && hh < NK;
+    float a[8];
+    float ss = 0.f;
+    if (ok) {
+      Eight<EI>::ld(isq ? q + t * q_ld + (int64_t)hh * d + i0 : k + t * k_ld + (int64_t)(hh - H) * d + i0, a);
+#pragma unroll
+      for (int i = 0; i < 8; i++) ss = fmaf(a[i], a[i], ss);
+    }
+    if (normed) {
+#pragma unroll
+      for (int o = LPH / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+    }
+    if (!ok) continue;
+    const E* nw = isq ? qn : kn;
+    if (nw) {
+      const float rs = 1.0f / sqrtf(ss / (float)d + eps);
+      float w[8];
+      Eight<E>::ld(nw + i0, w);
+#pragma unroll
+      for (int i = 0; i < 8; i++) a[i] = a[i] * rs * w[i];
+    }
+    if (turn) {
+#pragma unroll
+      for (int i = 0; i < 8; i += 2) {
+        const float n0 = a[i] * cs[i] - a[i + 1] * cs[i + 1];
+        a[i + 1] = a[i + 1] * cs[i] + a[i] * cs[i + 1];
+        a[i] = n0;
+      }
+    }
+    if (isq) {
+      if (temp) {
+        const float f = temp[hh];
+#pragma unroll
+        for (int i = 0; i < 8; i++) a[i] *= f;
+      }
+      Eight<float>::st(qo + (t * H + hh) * d + i0, a);
+    } else {
+      Eight<E>::st(row + (int64_t)(hh - H) * d + i0, a);
+    }
+  }
+  if (k)
+    for (int e = 8 * threadIdx.x; e < G * dv; e += 8 * blockDim.x) {
+      float a[8];
+      Eight<EI>::ld(v + t * v_ld + e, a);
+      Eight<E>::st(row + (int64_t)G * d + e, a);
+    }
 }
 
 // ------------------------------------------------------------------ attention
@@ -626,23 +645,32 @@ void qkv_norm_rope_store(bool in_bf16, bool bf16, const void* q, int64_t q_ld, c
   (void)num_rows;
   if (T <= 0) return;
   const size_t ei = in_bf16 ? 2 : 4, eo = bf16 ? 2 : 4;
-  auto even = [](const void* p, size_t eb) { return (uintptr_t)p % (2 * eb) == 0; };
-  const bool row2 = ((int64_t)G * (d + dv)) % 2 == 0;               // a row starts at an even element
-  if (!whole && (!table || layout != kHalf) && d % 2 == 0 && d <= 512 && q_ld % 2 == 0 && even(q, ei) && even(qn, eo) &&
-      even(kn, eo) && (!k || (k_ld % 2 == 0 && even(k, ei) && even(rows, eo) && row2))) {
-    const int heads = H + (k ? 2 * G : 0), nw = T > 64 ? 4 : (heads < 16 ? heads : 16);
-#define MA_PAIRS(EI, E, PL)                                                                                             \
-  qkv_store_pairs_k<EI, E, PL><<<T, 64 * nw, 0, st>>>((const EI*)q, q_ld, (const EI*)k, k_ld, (const EI*)v, v_ld,       \
-                                                      (const E*)qn, (const E*)kn, eps, table, dims, pos, slots, (E*)rows, \
-                                                      qo, temp, H, G, d, dv)
-#define MA_PL(EI, E)                        \
-  if (d <= 128) MA_PAIRS(EI, E, 1);         \
-  else if (d <= 256) MA_PAIRS(EI, E, 2);    \
-  else MA_PAIRS(EI, E, 4)
-    if (bf16 && in_bf16) { MA_PL(__bf16, __bf16); }
-    else if (bf16) { MA_PL(float, __bf16); }
-    else { MA_PL(float, float); }
-#undef MA_PL
+  auto wide = [](const void* p, int64_t ld, size_t eb) { return (uintptr_t)p % (8 * eb) == 0 && ld % 8 == 0; };
+  if (!whole && (!table || layout != kHalf) && d % 8 == 0 && d <= 512 && wide(q, q_ld, ei) && wide(qn, 0, eo) &&
+      wide(kn, 0, eo) && (!k || (dv % 8 == 0 && wide(k, k_ld, ei) && wide(v, v_ld, ei) && wide(rows, 0, eo)))) {
+    int lph = 1;
+    while (8 * lph < d) lph *= 2;
+    int nt = (H + (k ? G : 0)) * lph;                               // at most two passes over the heads for few tokens
+    nt = (nt + 63) / 64 * 64;
+    nt = T > 64 ? (nt > 256 ? 256 : nt) : (nt > 512 ? 512 : nt);
+#define MA_PAIRS(EI, E, L)                                                                                              \
+  qkv_store_pairs_k<EI, E, L><<<T, nt, 0, st>>>((const EI*)q, q_ld, (const EI*)k, k_ld, (const EI*)v, v_ld,             \
+                                                (const E*)qn, (const E*)kn, eps, table, dims, pos, slots, (E*)rows, qo, \
+                                                temp, H, G, d, dv)
+#define MA_L(EI, E)                      \
+  switch (lph) {                         \
+    case 1: MA_PAIRS(EI, E, 1); break;   \
+    case 2: MA_PAIRS(EI, E, 2); break;   \
+    case 4: MA_PAIRS(EI, E, 4); break;   \
+    case 8: MA_PAIRS(EI, E, 8); break;   \
+    case 16: MA_PAIRS(EI, E, 16); break; \
+    case 32: MA_PAIRS(EI, E, 32); break; \
+    default: MA_PAIRS(EI, E, 64);        \
+  }
+    if (bf16 && in_bf16) { MA_L(__bf16, __bf16) }
+    else if (bf16) { MA_L(float, __bf16) }
+    else { MA_L(float, float) }
+#undef MA_L
 #undef MA_PAIRS
     return;
   }

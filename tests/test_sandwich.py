@@ -445,18 +445,19 @@ def test_clamped_feed_forward(dev):
         assert (ff(h.to(dev)).double().cpu() - want).abs().max() < 1e-4 * max(1.0, float(want.abs().max()))
 
 
+@pytest.mark.parametrize("d,dv,dims", [(12, 10, 8), (16, 8, 6), (96, 24, 48), (128, 128, 128), (40, 16, 40), (8, 6, 2)])
 @pytest.mark.parametrize("act", [torch.float32, torch.bfloat16])
-def test_query_factor_and_head_gate(dev, act):
+def test_query_factor_and_head_gate(dev, act, d, dv, dims):
     from ipex_llm_amd.ops import maskattn as MA
     from ipex_llm_amd.ops.seqmix import rope_table
     g = torch.Generator().manual_seed(4)
-    T, H, G, d, dv = 11, 4, 2, 12, 10
+    T, H, G = 11, 6, 2
     y = torch.randn(T, H * d + G * (d + dv), generator=g).to(act)
     q, k, v = y[:, :H * d].view(T, H, d), y[:, H * d:(H + G) * d].view(T, G, d), y[:, (H + G) * d:].view(T, G, dv)
     qn, kn = (1 + 0.3 * torch.randn(d, generator=g)).to(act), (1 + 0.3 * torch.randn(d, generator=g)).to(act)
     temp = torch.rand(H, generator=g) + 0.5
-    rot = {"dims": 8, "base": 3000.0, "scaling": O.YARN}
-    tab = rope_table(64, 8, 3000.0, O.YARN)
+    rot = {"dims": dims, "base": 3000.0, "scaling": O.YARN}
+    tab = rope_table(64, dims, 3000.0, O.YARN)
     pos = torch.arange(20, 20 + T)
     rows = torch.zeros(2, 64, G * (d + dv), dtype=act, device=dev)
     yd = y.to(dev)
