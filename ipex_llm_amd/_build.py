@@ -99,9 +99,10 @@ TARGETS = {
     # (+ the streaming skinny-GEMM kernel their decode-size projections share with the dense decoders)
     "seqmix": ["hip/seqmix.hip", "hip/blockmix_elem.hip", "hip/blockmix_attn.hip", "hip/blockmix_moe.hip",
                "hip/ssm.hip", "hip/maskattn.hip", "hip/gatedmix.hip", "hip/statemix.hip",
-               "hip/statemix_scan.hip", "hip/statemix_chunk.hip", "hip/dense_gemv.hip", "torch/ops_seqmix.cpp",
-               "torch/ops_blockmix.cpp", "torch/ops_ssm.cpp", "torch/ops_maskattn.cpp", "torch/ops_gatedmix.cpp", "torch/ops_statemix.cpp",
-               "torch/ops_dense.cpp",
+               "hip/statemix_scan.hip", "hip/statemix_chunk.hip", "hip/chanmix.hip", "hip/chanmix_scan.hip",
+               "hip/chanmix_chunk.hip", "hip/dense_gemv.hip", "torch/ops_seqmix.cpp",
+               "torch/ops_blockmix.cpp", "torch/ops_ssm.cpp", "torch/ops_maskattn.cpp", "torch/ops_gatedmix.cpp",
+               "torch/ops_statemix.cpp", "torch/ops_chanmix.cpp", "torch/ops_dense.cpp",
                "runtime/scheduler.cpp"],
 }
 

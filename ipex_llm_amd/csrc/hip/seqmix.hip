@@ -195,14 +195,23 @@ template <typename E> struct Chunk4;
 template <> struct Chunk4<float> { typedef uint4 type; };
 template <> struct Chunk4<__bf16> { typedef uint2 type; };
 
+// 1 / (denominator including the sink's exp(sink_h)) for the sum L relative to the maximum M, times what brings a sum
+// relative to M to the joint maximum
+__device__ __forceinline__ float with_sink(float M, float L, const float* sink, int h) {
+  if (!sink) return 1.0f / L;
+  const float s = sink[h], m = fmaxf(M, s), f = expf(M - m);
+  return f / (L * f + expf(s - m));
+}
+
 template <typename E, int RC, int HB>
 __global__ void __launch_bounds__(256) latent_attn_k(const E* __restrict__ q_lat, const E* __restrict__ q_rot,
                                                     int64_t qr_st, int64_t qr_sh, const E* __restrict__ rows, int bs,
                                                     const int32_t* __restrict__ bt, int bt_w,
                                                     const int32_t* __restrict__ seq_of, const int64_t* __restrict__ pos,
                                                     float scale, const E* __restrict__ gate, int64_t g_st,
-                                                    E* __restrict__ out, float* __restrict__ part, int H, int r, int dr,
-                                                    int KT, int DP, int window) {
+                                                    const float* __restrict__ sink, E* __restrict__ out,
+                                                    float* __restrict__ part, int H, int r, int dr, int KT, int DP,
+                                                    int window) {
   extern __shared__ __align__(16) unsigned char smem[];
   const int D = r + dr, D4 = (D + 3) & ~3;
   const int nsplit = gridDim.z, zs = blockIdx.z;
@@ -383,7 +392,7 @@ __global__ void __launch_bounds__(256) latent_attn_k(const E* __restrict__ q_lat
       float* pp = part + (((int64_t)t * H + h0 + h) * nsplit + zs) * (r + 2);
       pp[c] = c < r ? O : (c == r ? M : L);
     } else if (c < r) {
-      float v = O / L;
+      float v = O * with_sink(M, L, sink, h0 + h);
       if (gate) v *= 1.0f / (1.0f + expf(-ldf(gate + (int64_t)t * g_st + h0 + h)));
       stf(out + ((int64_t)t * H + h0 + h) * r + c, v);
     }
@@ -408,8 +417,9 @@ __global__ void __launch_bounds__(256) latent_attn_mfma_k(const __bf16* __restri
                                                          const int32_t* __restrict__ seq_of,
                                                          const int64_t* __restrict__ pos, float scale,
                                                          const __bf16* __restrict__ gate, int64_t g_st,
-                                                         __bf16* __restrict__ out, float* __restrict__ part, int H, int r,
-                                                         int dr, int DP, int window) {
+                                                         const float* __restrict__ sink, __bf16* __restrict__ out,
+                                                         float* __restrict__ part, int H, int r, int dr, int DP,
+                                                         int window) {
   typedef __bf16 E;
   constexpr int KT = 16;
   extern __shared__ __align__(16) unsigned char smem[];
@@ -585,7 +595,7 @@ __global__ void __launch_bounds__(256) latent_attn_mfma_k(const __bf16* __restri
       float* pp = part + (((int64_t)t * H + h0 + h) * nsplit + zs) * (r + 2);
       pp[c] = c < r ? O : (c == r ? M : L);
     } else if (c < r) {
-      float v = O / L;
+      float v = O * with_sink(M, L, sink, h0 + h);
       if (gate) v *= 1.0f / (1.0f + expf(-ldf(gate + (int64_t)t * g_st + h0 + h)));
       stf(out + ((int64_t)t * H + h0 + h) * r + c, v);
     }
@@ -596,8 +606,8 @@ __global__ void __launch_bounds__(256) latent_attn_mfma_k(const __bf16* __restri
 // merge of the key splits: part [T, H, nsplit, r + 2] -> out [T, H, r]
 template <typename E>
 __global__ void __launch_bounds__(128) latent_attn_combine_k(const float* __restrict__ part, const E* __restrict__ gate,
-                                                            int64_t g_st, E* __restrict__ out, int H, int r,
-                                                            int nsplit) {
+                                                            int64_t g_st, const float* __restrict__ sink,
+                                                            E* __restrict__ out, int H, int r, int nsplit) {
   __shared__ float wz[64];                                          // exp(m_z - M) / L * gate, nsplit <= 64
   const int64_t t = blockIdx.x;
   const int h = blockIdx.y;
@@ -609,7 +619,7 @@ __global__ void __launch_bounds__(128) latent_attn_combine_k(const float* __rest
     const float e = mz == -INFINITY ? 0.f : expf(mz - M);
     const float L = wave_sum(z < nsplit ? pp[(int64_t)z * (r + 2) + r + 1] * e : 0.f);
     const float g = gate ? 1.0f / (1.0f + expf(-ldf(gate + t * g_st + h))) : 1.0f;
-    wz[z] = e / L * g;
+    wz[z] = e * with_sink(M, L, sink, h) * g;
   }
   __syncthreads();
   for (int c = threadIdx.x; c < r; c += blockDim.x) {
@@ -628,7 +638,7 @@ __global__ void __launch_bounds__(128) latent_attn_combine_k(const float* __rest
 template <typename E>
 __global__ void __launch_bounds__(256) causal_softmax_k(float* __restrict__ sc, int64_t ld, const int64_t* __restrict__ pos,
                                                        int H, float scale, int L, E* __restrict__ hi, E* __restrict__ lo,
-                                                       int64_t key0, int window) {
+                                                       int64_t key0, int window, const float* __restrict__ sink) {
   __shared__ float red[16];
   const int64_t row = blockIdx.x;
   const int64_t p = pos[row / H];
@@ -636,7 +646,8 @@ __global__ void __launch_bounds__(256) causal_softmax_k(float* __restrict__ sc, 
   const int nk = (int)max((int64_t)0, min((int64_t)L, p - key0 + 1));
   const int j0 = window > 0 ? (int)max((int64_t)0, min((int64_t)nk, p - window + 1 - key0)) : 0;
   float* s = sc + row * ld;
-  float mx = -INFINITY;
+  const float sk = sink ? sink[row % H] : -INFINITY;
+  float mx = sk;
   for (int j = j0 + threadIdx.x; j < nk; j += blockDim.x) mx = fmaxf(mx, s[j] * scale);
   mx = wave_max(mx);
   __syncthreads();
@@ -649,7 +660,7 @@ __global__ void __launch_bounds__(256) causal_softmax_k(float* __restrict__ sc, 
     s[j] = e;
     sum += e;
   }
-  const float inv = 1.0f / block_sum(sum, red);
+  const float inv = 1.0f / (block_sum(sum, red) + (sink ? expf(sk - mx) : 0.f));
   for (int j = threadIdx.x; j < L; j += blockDim.x) {
     const float w = j >= j0 && j < nk ? s[j] * inv : 0.f;
     if (hi) {
@@ -839,10 +850,11 @@ __global__ void __launch_bounds__(256) mlstm_scan_k(const E* __restrict__ q, int
   }
 }
 
+// gate: sigmoid, or SiLU (silu != 0)
 template <typename E>
 __global__ void __launch_bounds__(64) head_rms_gate_k(const float* __restrict__ hh, const E* __restrict__ nw,
                                                      const E* __restrict__ gate, int64_t g_ld, E* __restrict__ out,
-                                                     int H, int dv, float eps) {
+                                                     int H, int dv, float eps, int silu) {
   const int64_t t = blockIdx.x;
   const int h = blockIdx.y;
   const float* in = hh + (t * H + h) * dv;
@@ -850,7 +862,7 @@ __global__ void __launch_bounds__(64) head_rms_gate_k(const float* __restrict__ 
   for (int c = threadIdx.x; c < dv; c += 64) q += in[c] * in[c];
   const float rs = 1.0f / sqrtf(wave_sum(q) / (float)dv + eps);
   for (int c = threadIdx.x; c < dv; c += 64) {
-    const float g = 1.0f / (1.0f + expf(-ldf(gate + t * g_ld + h * dv + c)));
+    const float z = ldf(gate + t * g_ld + h * dv + c), g = (silu ? z : 1.0f) / (1.0f + expf(-z));
     stf(out + (t * H + h) * dv + c, in[c] * rs * ldf(nw + h * dv + c) * g);
   }
 }
@@ -993,8 +1005,8 @@ int latent_attention_splits(bool bf16, int T, int H, int r, int dr, int max_ctx)
 
 void latent_attention(bool bf16, const void* q_lat, const void* q_rot, int64_t qr_st, int64_t qr_sh, const void* rows,
                       int bs, const int32_t* block_tables, int bt_width, const int32_t* seq_of, const int64_t* pos,
-                      float scale, const void* gate, int64_t g_st, void* out, float* part, int nsplit, int T, int H,
-                      int r, int dr, int window, hipStream_t st) {
+                      float scale, const void* gate, int64_t g_st, const float* sink, void* out, float* part, int nsplit,
+                      int T, int H, int r, int dr, int window, hipStream_t st) {
   if (T <= 0) return;
   const int rc = (r + 63) / 64;
   int KT = 0, NW = 0, hb = 8;
@@ -1006,7 +1018,7 @@ void latent_attention(bool bf16, const void* q_lat, const void* q_rot, int64_t q
 #define SM_ATTN_M(RC, HBV)                                                                                            \
   hipLaunchKernelGGL((latent_attn_mfma_k<RC, HBV>), grid, block, lds, st, (const __bf16*)q_lat, (const __bf16*)q_rot,  \
                      qr_st, qr_sh, (const __bf16*)rows, bs, block_tables, bt_width, seq_of, pos, scale,                \
-                     (const __bf16*)gate, g_st, (__bf16*)out, part, H, r, dr, DP, window)
+                     (const __bf16*)gate, g_st, sink, (__bf16*)out, part, H, r, dr, DP, window)
       if (hb == 8) {
         if (rc <= 1) { SM_ATTN_M(1, 8); }
         else if (rc <= 2) { SM_ATTN_M(2, 8); }
@@ -1019,7 +1031,7 @@ void latent_attention(bool bf16, const void* q_lat, const void* q_rot, int64_t q
 #undef SM_ATTN_M
       if (nsplit > 1)
         hipLaunchKernelGGL(latent_attn_combine_k<__bf16>, dim3(T, H), dim3(128), 0, st, part, (const __bf16*)gate, g_st,
-                           (__bf16*)out, H, r, nsplit);
+                           sink, (__bf16*)out, H, r, nsplit);
       return;
     }
   }
@@ -1030,8 +1042,8 @@ void latent_attention(bool bf16, const void* q_lat, const void* q_rot, int64_t q
 #define SM_ATTN(RC, HBV)                                                                                              \
   SM_DISPATCH(bf16, hipLaunchKernelGGL((latent_attn_k<E, RC, HBV>), grid, block, lds, st, (const E*)q_lat,             \
                                        (const E*)q_rot, qr_st, qr_sh, (const E*)rows, bs, block_tables, bt_width,      \
-                                       seq_of, pos, scale, (const E*)gate, g_st, (E*)out, part, H, r, dr, KT, DP,      \
-                                       window))
+                                       seq_of, pos, scale, (const E*)gate, g_st, sink, (E*)out, part, H, r, dr, KT,    \
+                                       DP, window))
   if (hb == 8) {
     if (rc <= 1) { SM_ATTN(1, 8); }
     else if (rc <= 2) { SM_ATTN(2, 8); }
@@ -1044,19 +1056,19 @@ void latent_attention(bool bf16, const void* q_lat, const void* q_rot, int64_t q
 #undef SM_ATTN
   if (nsplit > 1) {
     SM_DISPATCH(bf16, hipLaunchKernelGGL(latent_attn_combine_k<E>, dim3(T, H), dim3(128), 0, st, part, (const E*)gate,
-                                         g_st, (E*)out, H, r, nsplit));
+                                         g_st, sink, (E*)out, H, r, nsplit));
   }
 }
 
 void causal_softmax(bool bf16, float* sc, int64_t ld, const int64_t* pos, int H, float scale, int64_t R, int L, void* hi,
-                    void* lo, int64_t key0, int window, hipStream_t st) {
+                    void* lo, int64_t key0, int window, const float* sink, hipStream_t st) {
   if (R <= 0 || L <= 0) return;
   if (bf16) {
     hipLaunchKernelGGL(causal_softmax_k<__bf16>, dim3((unsigned)R), dim3(256), 0, st, sc, ld, pos, H, scale, L,
-                       (__bf16*)hi, (__bf16*)lo, key0, window);
+                       (__bf16*)hi, (__bf16*)lo, key0, window, sink);
   } else {
     hipLaunchKernelGGL(causal_softmax_k<float>, dim3((unsigned)R), dim3(256), 0, st, sc, ld, pos, H, scale, L,
-                       (float*)nullptr, (float*)nullptr, key0, window);
+                       (float*)nullptr, (float*)nullptr, key0, window, sink);
   }
 }
 
@@ -1087,10 +1099,10 @@ void mlstm_scan(bool bf16, const void* q, int64_t q_ld, const void* k, int64_t k
 }
 
 void head_rms_gate(bool bf16, const float* h, const void* norm_w, const void* gate, int64_t g_ld, void* out, int T,
-                   int H, int dv, float eps, hipStream_t st) {
+                   int H, int dv, float eps, bool silu, hipStream_t st) {
   if (T <= 0) return;
   SM_DISPATCH(bf16, hipLaunchKernelGGL(head_rms_gate_k<E>, dim3(T, H), dim3(64), 0, st, h, (const E*)norm_w,
-                                       (const E*)gate, g_ld, (E*)out, H, dv, eps));
+                                       (const E*)gate, g_ld, (E*)out, H, dv, eps, silu ? 1 : 0));
 }
 
 void glu_act(bool bf16, const void* gu, void* out, int64_t T, int64_t I, int act, hipStream_t st) {

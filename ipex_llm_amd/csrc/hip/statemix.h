@@ -29,12 +29,17 @@ void add_normed_experts(bool bf16, float* x, const float* rows, const int32_t* i
 // out = o / rms(o) w sigmoid(gate), o f32 [T, C]
 void rms_sigmoid_gate(bool bf16, const float* o, const void* w, const void* gate, int64_t g_ld, void* out, int T, int C,
                       float eps, hipStream_t st);
-// softmax over all E <= 512, choice by s + corr inside the best ``keep`` of ``groups`` groups, weights s
-void route_groups(const float* z, const float* corr, int T, int E, int top, int groups, int keep, int32_t* idx, float* w,
-                  hipStream_t st);
+// E <= 512 scores s (softmax over all, or sigmoid); choice by s + corr inside the best ``keep`` of ``groups`` groups; a
+// group's score: its largest corrected score, or the sum of its two largest; weights s, or scale s / (their sum + 1e-20)
+struct RouteRule {
+  bool sigmoid, best_two, renorm;
+  float scale;
+};
+void route_groups(const float* z, const float* corr, RouteRule rule, int T, int E, int top, int groups, int keep,
+                  int32_t* idx, float* w, hipStream_t st);
 // the same from the router's input rows h [T, W] (activation type) and weights rw f32 [E, W]
-void router(bool bf16, const void* h, const float* rw, const float* corr, int T, int W, int E, int top, int groups,
-            int keep, int32_t* idx, float* w, hipStream_t st);
+void router(bool bf16, const void* h, const float* rw, const float* corr, RouteRule rule, int T, int W, int E, int top,
+            int groups, int keep, int32_t* idx, float* w, hipStream_t st);
 
 // ---- recurrences (statemix_scan.hip)
 constexpr int kScanMaxDim = 512;

@@ -9,7 +9,7 @@
 //                      of a token's expert rows (identity experts add their
 //                      weight times the input)
 //   RMS + sigmoid gate over the whole row
-//   group routing      one wave per token: softmax over all router outputs,
+//   group routing      one wave per token: softmax over all router outputs (or sigmoids),
 //                      corrected scores and the groups' best ones in LDS, the
 //                      kept groups by rank, then the winners one after another;
 //                      for few tokens the same launch forms the logits
@@ -212,8 +212,8 @@ __device__ __forceinline__ void wave_sync() {
   __builtin_amdgcn_wave_barrier();
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 }
-__device__ void route_wave(const float* z, const float* __restrict__ corr, int E, int top, int groups, int keep,
-                           int32_t* __restrict__ idx, float* __restrict__ w, int64_t t, float* cs, float* best) {
+__device__ void route_wave(const float* z, const float* __restrict__ corr, RouteRule rule, int E, int top, int groups,
+                           int keep, int32_t* __restrict__ idx, float* __restrict__ w, int64_t t, float* cs, float* best) {
   const int lane = threadIdx.x & 63;
   float s[kPerLane], c[kPerLane];
   float mx = -INFINITY;
@@ -223,18 +223,24 @@ __device__ void route_wave(const float* z, const float* __restrict__ corr, int E
     s[i] = e < E ? z[e] : -INFINITY;
     mx = fmaxf(mx, s[i]);
   }
-  mx = wave_max(mx);
-  float sum = 0.f;
+  if (rule.sigmoid) {
 #pragma unroll
-  for (int i = 0; i < kPerLane; i++) {
-    s[i] = lane + 64 * i < E ? expf(s[i] - mx) : 0.f;
-    sum += s[i];
+    for (int i = 0; i < kPerLane; i++) s[i] = lane + 64 * i < E ? 1.0f / (1.0f + expf(-s[i])) : 0.f;
+  } else {
+    mx = wave_max(mx);
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < kPerLane; i++) {
+      s[i] = lane + 64 * i < E ? expf(s[i] - mx) : 0.f;
+      sum += s[i];
+    }
+    const float inv = 1.0f / wave_sum(sum);
+#pragma unroll
+    for (int i = 0; i < kPerLane; i++) s[i] *= inv;
   }
-  const float inv = 1.0f / wave_sum(sum);
 #pragma unroll
   for (int i = 0; i < kPerLane; i++) {
     const int e = lane + 64 * i;
-    s[i] *= inv;
     c[i] = e < E ? s[i] + (corr ? corr[e] : 0.f) : -INFINITY;
     if (e < E) cs[e] = c[i];
   }
@@ -242,9 +248,13 @@ __device__ void route_wave(const float* z, const float* __restrict__ corr, int E
     const int gs = E / groups;
     wave_sync();
     for (int g = lane; g < groups; g += 64) {
-      float b = -INFINITY;
-      for (int j = 0; j < gs; j++) b = fmaxf(b, cs[g * gs + j]);
-      best[g] = b;
+      float b = -INFINITY, b2 = -INFINITY;
+      for (int j = 0; j < gs; j++) {
+        const float v = cs[g * gs + j];
+        b2 = fmaxf(b2, fminf(b, v));
+        b = fmaxf(b, v);
+      }
+      best[g] = rule.best_two && gs > 1 ? b + b2 : b;
     }
     wave_sync();
     bool kept[kPerLane];
@@ -269,6 +279,7 @@ __device__ void route_wave(const float* z, const float* __restrict__ corr, int E
       if (e < E && best[e / gs] == 0.f) c[i] = -INFINITY;
     }
   }
+  float total = 0.f;
   for (int k = 0; k < top; k++) {
     float bv = -INFINITY;
     int be = 0x7fffffff;
@@ -296,26 +307,42 @@ __device__ void route_wave(const float* z, const float* __restrict__ corr, int E
     for (int i = 0; i < kPerLane; i++)
       if (lane + 64 * i == be) {
         idx[t * top + k] = be;
-        w[t * top + k] = s[i];
+        if (!rule.renorm) w[t * top + k] = s[i];
         c[i] = -INFINITY;
       }
+    if (rule.renorm) {                                              // the winner's score to every lane
+      float sv = 0.f;
+#pragma unroll
+      for (int i = 0; i < kPerLane; i++)
+        if (lane + 64 * i == be) sv = s[i];
+      if (lane == 0) cs[k] = 0.f;
+      wave_sync();
+      if (!none && (be & 63) == lane) cs[k] = sv;
+      wave_sync();
+      total += cs[k];
+    }
+  }
+  if (rule.renorm) {
+    const float f = rule.scale / (total + 1e-20f);
+    for (int k = lane; k < top; k += 64) w[t * top + k] = cs[k] * f;
   }
 }
 
-__global__ void __launch_bounds__(64) route_groups_k(const float* __restrict__ z, const float* __restrict__ corr, int E,
-                                                    int top, int groups, int keep, int32_t* __restrict__ idx,
+__global__ void __launch_bounds__(64) route_groups_k(const float* __restrict__ z, const float* __restrict__ corr,
+                                                    RouteRule rule, int E, int top, int groups, int keep, int32_t* __restrict__ idx,
                                                     float* __restrict__ w) {
   __shared__ float cs[64 * kPerLane];                               // corrected scores
   __shared__ float best[64 * kPerLane];                             // per group; kept ones become 1, others 0
   const int64_t t = blockIdx.x;
-  route_wave(z + t * E, corr, E, top, groups, keep, idx, w, t, cs, best);
+  route_wave(z + t * E, corr, rule, E, top, groups, keep, idx, w, t, cs, best);
 }
 
 // few tokens: the logits as well (f32 products of the router with the token's row, a wave per router output), then the
 // first wave routes
 template <typename E, int V>
 __global__ void __launch_bounds__(1024) router_k(const E* __restrict__ h, const float* __restrict__ rw,
-                                                const float* __restrict__ corr, int W, int NE, int top, int groups, int keep,
+                                                const float* __restrict__ corr, RouteRule rule, int W, int NE, int top,
+                                                int groups, int keep,
                                                 int32_t* __restrict__ idx, float* __restrict__ w) {
   __shared__ float cs[64 * kPerLane], best[64 * kPerLane], z[64 * kPerLane];
   const int64_t t = blockIdx.x;
@@ -334,7 +361,7 @@ __global__ void __launch_bounds__(1024) router_k(const E* __restrict__ h, const 
     if (lane == 0) z[e] = s;
   }
   __syncthreads();
-  if (wv == 0) route_wave(z, corr, NE, top, groups, keep, idx, w, t, cs, best);
+  if (wv == 0) route_wave(z, corr, rule, NE, top, groups, keep, idx, w, t, cs, best);
 }
 
 int row_threads(int W, int V) {
@@ -398,17 +425,17 @@ void rms_sigmoid_gate(bool bf16, const float* o, const void* w, const void* gate
     rms_sigmoid_gate_k<float><<<T, nt, 0, st>>>(o, (const float*)w, (const float*)gate, g_ld, (float*)out, C, eps);
 }
 
-void route_groups(const float* z, const float* corr, int T, int E, int top, int groups, int keep, int32_t* idx, float* w,
-                  hipStream_t st) {
+void route_groups(const float* z, const float* corr, RouteRule rule, int T, int E, int top, int groups, int keep,
+                  int32_t* idx, float* w, hipStream_t st) {
   if (T <= 0) return;
-  route_groups_k<<<T, 64, 0, st>>>(z, corr, E, top, groups, keep, idx, w);
+  route_groups_k<<<T, 64, 0, st>>>(z, corr, rule, E, top, groups, keep, idx, w);
 }
 
-void router(bool bf16, const void* h, const float* rw, const float* corr, int T, int W, int E, int top, int groups,
-            int keep, int32_t* idx, float* w, hipStream_t st) {
+void router(bool bf16, const void* h, const float* rw, const float* corr, RouteRule rule, int T, int W, int E, int top,
+            int groups, int keep, int32_t* idx, float* w, hipStream_t st) {
   if (T <= 0) return;
   const int nt = 64 * (E < 16 ? E : 16);
-#define CALL(EL, V) (router_k<EL, V><<<T, nt, 0, st>>>((const EL*)h, rw, corr, W, E, top, groups, keep, idx, w))
+#define CALL(EL, V) (router_k<EL, V><<<T, nt, 0, st>>>((const EL*)h, rw, corr, rule, W, E, top, groups, keep, idx, w))
   if (bf16) { SX_V(W, CALL(__bf16, 1), CALL(__bf16, 4)) } else { SX_V(W, CALL(float, 1), CALL(float, 4)) }
 #undef CALL
 }

@@ -19,6 +19,7 @@
 //                      run again
 //
 // Activations are bf16 or f32 (template E); accumulation is always f32.
+#include "split_tile.h"
 #include "statemix.h"
 
 #include <math.h>
@@ -207,43 +208,9 @@ void launch_scan(const EQ* q, int64_t q_ld, const EQ* k, int64_t k_ld, const EQ*
 }
 
 // ------------------------------------------------------------------ gates of the linear recurrent unit
-typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
-typedef float f32x4 __attribute__((ext_vector_type(4)));
-
 // a workgroup: TM tokens x 64 output channels of one block, both gates; wave w owns channels 16 w .. 16 w + 15.
 // K goes by 64; inside a step of 32 lane group g holds k = 8 g .. 8 g + 7 (tokens' values and weights alike, so the
 // f32 products may take them one after another)
-template <typename E> struct Parts { static constexpr int N = 1; };
-template <> struct Parts<__bf16> { static constexpr int N = 3; };
-
-// 8 consecutive weights of a row from index kk on, zeros from n on (vec: n is a multiple of 8, rows are 16-byte aligned)
-template <typename E> struct Frag {
-  E __attribute__((aligned(16))) v[8];
-  __device__ __forceinline__ void load(const E* w, int kk, int n, bool vec) {
-    if (vec && kk < n) {
-      const uint4* s = (const uint4*)(w + kk);
-      uint4* d = (uint4*)v;
-#pragma unroll
-      for (int i = 0; i < (int)(8 * sizeof(E) / 16); i++) d[i] = s[i];
-    } else {
-#pragma unroll
-      for (int j = 0; j < 8; j++) v[j] = kk + j < n ? w[kk + j] : (E)0.f;
-    }
-  }
-  __device__ __forceinline__ bf16x8 v8() const { return *(const bf16x8*)v; }
-};
-
-// an f32 value as the parts of E whose sum it is
-template <int N> __device__ __forceinline__ void stage(float (*us)[N], int at, float v) { us[0][at] = v; }
-template <int N> __device__ __forceinline__ void stage(__bf16 (*us)[N], int at, float v) {
-  const __bf16 hi = (__bf16)v;
-  const float r1 = v - (float)hi;
-  const __bf16 mid = (__bf16)r1;
-  us[0][at] = hi;
-  us[1][at] = mid;
-  us[2][at] = (__bf16)(r1 - (float)mid);
-}
-
 template <typename E, int TM>
 __global__ void __launch_bounds__(256) rglru_gates_k(const float* __restrict__ u, const E* __restrict__ w_r,
                                                     const float* __restrict__ b_r, const E* __restrict__ w_i,

@@ -116,9 +116,16 @@ int64_t sm_latent_attention_fits(bool bf16, int64_t H, int64_t r, int64_t dr) {
   return illm::sm::latent_attention_plan(bf16, (int)H, (int)r, (int)dr, &kt, &nw, &hb);
 }
 
+const float* sink_ptr(const c10::optional<Tensor>& sink, int64_t H, const char* what) {
+  if (!sink.has_value() || !sink->defined()) return nullptr;
+  TORCH_CHECK(sink->is_cuda() && sink->scalar_type() == at::kFloat && sink->is_contiguous() && sink->numel() == H, what,
+              ": sink f32 [H]");
+  return sink->data_ptr<float>();
+}
+
 Tensor sm_latent_attention(const Tensor& q_lat, const Tensor& q_rot, const Tensor& rows, const Tensor& block_tables,
                            const Tensor& seq_of, const Tensor& pos, double scale, const c10::optional<Tensor>& gate,
-                           int64_t max_ctx, bool act_f32, int64_t window) {
+                           int64_t max_ctx, bool act_f32, int64_t window, const c10::optional<Tensor>& sink) {
   c10::DeviceGuard g(q_lat.device());
   TORCH_CHECK(q_lat.is_cuda() && q_lat.dim() == 3 && is_act(q_lat) && q_lat.is_contiguous(),
               "sm_latent_attention: q_lat [T, H, r] contiguous");
@@ -140,6 +147,7 @@ Tensor sm_latent_attention(const Tensor& q_lat, const Tensor& q_rot, const Tenso
   check_idx(seq_of, at::kInt, T, "sm_latent_attention: seq_of int32 [T]");
   check_idx(pos, at::kLong, T, "sm_latent_attention: pos int64 [T]");
   TORCH_CHECK(r >= 1 && r <= 512, "sm_latent_attention: latent size must be 1..512");
+  const float* sp = sink_ptr(sink, H, "sm_latent_attention");
   const void* gp = nullptr;
   int64_t gst = 0;
   if (gate.has_value() && gate->defined()) {
@@ -162,14 +170,14 @@ Tensor sm_latent_attention(const Tensor& q_lat, const Tensor& q_rot, const Tenso
   illm::sm::latent_attention(bf(q_lat), q_lat.data_ptr(), q_rot.data_ptr(), q_rot.stride(0), q_rot.stride(1),
                              rows.data_ptr(), (int)rows.size(1), block_tables.data_ptr<int32_t>(),
                              (int)block_tables.size(1), seq_of.data_ptr<int32_t>(), pos.data_ptr<int64_t>(), (float)scale,
-                             gp, gst, out.data_ptr(), nsplit > 1 ? part.data_ptr<float>() : nullptr, nsplit, (int)T,
+                             gp, gst, sp, out.data_ptr(), nsplit > 1 ? part.data_ptr<float>() : nullptr, nsplit, (int)T,
                              (int)H, (int)r, (int)dr, (int)window, stream());
   return out;
 }
 
 // scores f32 [R, L] (R = tokens x H rows) -> causal softmax weights; bf16 pair (hi, lo) or in place (f32)
 std::tuple<Tensor, Tensor> sm_causal_softmax(Tensor& scores, const Tensor& pos, int64_t H, double scale, bool act_f32,
-                                             int64_t key0, int64_t window) {
+                                             int64_t key0, int64_t window, const c10::optional<Tensor>& sink) {
   c10::DeviceGuard g(scores.device());
   TORCH_CHECK(scores.is_cuda() && scores.dim() == 2 && scores.scalar_type() == at::kFloat && scores.is_contiguous(),
               "sm_causal_softmax: scores f32 [R, L] contiguous");
@@ -184,7 +192,7 @@ std::tuple<Tensor, Tensor> sm_causal_softmax(Tensor& scores, const Tensor& pos, 
   }
   illm::sm::causal_softmax(!act_f32, scores.data_ptr<float>(), L, pos.data_ptr<int64_t>(), (int)H, (float)scale, R, (int)L,
                            act_f32 ? nullptr : hi.data_ptr(), act_f32 ? nullptr : lo.data_ptr(), key0, (int)window,
-                           stream());
+                           sink_ptr(sink, H, "sm_causal_softmax"), stream());
   if (act_f32) return {scores, scores};
   return {hi, lo};
 }
@@ -228,7 +236,7 @@ Tensor sm_mlstm_scan(const Tensor& q, const Tensor& k, const Tensor& v, const Te
   return out;
 }
 
-Tensor sm_head_rms_gate(const Tensor& h, const Tensor& norm_w, const Tensor& gate, double eps, bool act_f32) {
+Tensor sm_head_rms_gate(const Tensor& h, const Tensor& norm_w, const Tensor& gate, double eps, bool act_f32, bool silu) {
   c10::DeviceGuard g(h.device());
   TORCH_CHECK(h.is_cuda() && h.dim() == 3 && h.scalar_type() == at::kFloat && h.is_contiguous(),
               "sm_head_rms_gate: h f32 [T, H, dv]");
@@ -241,7 +249,7 @@ Tensor sm_head_rms_gate(const Tensor& h, const Tensor& norm_w, const Tensor& gat
               "sm_head_rms_gate: gate [T, H * dv]");
   Tensor out = at::empty({T, H * dv}, norm_w.options());
   illm::sm::head_rms_gate(bf(norm_w), h.data_ptr<float>(), norm_w.data_ptr(), gate.data_ptr(), gate.stride(0),
-                          out.data_ptr(), (int)T, (int)H, (int)dv, (float)eps, stream());
+                          out.data_ptr(), (int)T, (int)H, (int)dv, (float)eps, silu, stream());
   return out;
 }
 
@@ -276,13 +284,13 @@ TORCH_LIBRARY_FRAGMENT(ipex_llm_amd, m) {
   m.def("sm_latent_kv_store(Tensor dkv, Tensor norm_w, float eps, int rank, Tensor table, Tensor pos, Tensor slots, "
         "Tensor(a!) rows) -> ()");
   m.def("sm_latent_attention(Tensor q_lat, Tensor q_rot, Tensor rows, Tensor block_tables, Tensor seq_of, Tensor pos, "
-        "float scale, Tensor? gate, int max_ctx, bool act_f32, int window=0) -> Tensor");
+        "float scale, Tensor? gate, int max_ctx, bool act_f32, int window=0, Tensor? sink=None) -> Tensor");
   m.def("sm_latent_attention_fits(bool bf16, int H, int r, int dr) -> int");
   m.def("sm_mlstm_scan(Tensor q, Tensor k, Tensor v, Tensor ipre, Tensor fpre, Tensor ib, Tensor fb, float cap, "
         "Tensor(a!) S, Tensor(b!) n, Tensor(c!) m, Tensor cu, Tensor slots, Tensor pos, int max_q) -> Tensor");
-  m.def("sm_causal_softmax(Tensor(a!) scores, Tensor pos, int H, float scale, bool act_f32, int key0=0, int window=0) "
-        "-> (Tensor, Tensor)");
-  m.def("sm_head_rms_gate(Tensor h, Tensor norm_w, Tensor gate, float eps, bool act_f32) -> Tensor");
+  m.def("sm_causal_softmax(Tensor(a!) scores, Tensor pos, int H, float scale, bool act_f32, int key0=0, int window=0, "
+        "Tensor? sink=None) -> (Tensor, Tensor)");
+  m.def("sm_head_rms_gate(Tensor h, Tensor norm_w, Tensor gate, float eps, bool act_f32, bool silu=False) -> Tensor");
   m.def("sm_glu_gelu(Tensor gu) -> Tensor");
   m.def("sm_glu_act(Tensor gu, int act) -> Tensor");
 }

@@ -140,7 +140,8 @@ Tensor sx_rms_sigmoid_gate(const Tensor& o, const Tensor& w, const Tensor& gate,
   return out;
 }
 
-std::tuple<Tensor, Tensor> sx_route_groups(const Tensor& z, const OptT& corr, int64_t top, int64_t groups, int64_t keep) {
+std::tuple<Tensor, Tensor> sx_route_groups(const Tensor& z, const OptT& corr, int64_t top, int64_t groups, int64_t keep,
+                                           bool sigmoid, bool best_two, bool renorm, double scale) {
   c10::DeviceGuard g(z.device());
   TORCH_CHECK(z.is_cuda() && z.dim() == 2 && z.scalar_type() == at::kFloat && z.is_contiguous(),
               "sx_route_groups: logits f32 [T, E] contiguous");
@@ -150,13 +151,14 @@ std::tuple<Tensor, Tensor> sx_route_groups(const Tensor& z, const OptT& corr, in
               "sx_route_groups: E <= 512, equal groups, 1 <= top <= outputs of the kept groups");
   TORCH_CHECK(!has(corr) || vec(*corr, at::kFloat, E), "sx_route_groups: correction f32 [E]");
   Tensor idx = at::empty({T, top}, z.options().dtype(at::kInt)), w = at::empty({T, top}, z.options());
-  illm::sx::route_groups(z.data_ptr<float>(), has(corr) ? corr->data_ptr<float>() : nullptr, (int)T, (int)E, (int)top,
-                         (int)groups, (int)keep, idx.data_ptr<int32_t>(), w.data_ptr<float>(), stream());
+  illm::sx::route_groups(z.data_ptr<float>(), has(corr) ? corr->data_ptr<float>() : nullptr,
+                         {sigmoid, best_two, renorm, (float)scale}, (int)T, (int)E, (int)top, (int)groups,
+                         (int)keep, idx.data_ptr<int32_t>(), w.data_ptr<float>(), stream());
   return {idx, w};
 }
 
 std::tuple<Tensor, Tensor> sx_router(const Tensor& h, const Tensor& rw, const OptT& corr, int64_t top, int64_t groups,
-                                     int64_t keep) {
+                                     int64_t keep, bool sigmoid, bool best_two, bool renorm, double scale) {
   c10::DeviceGuard g(h.device());
   TORCH_CHECK(h.is_cuda() && h.dim() == 2 && is_act(h) && h.is_contiguous(), "sx_router: h [T, W] contiguous");
   const int64_t T = h.size(0), W = h.size(1), E = rw.dim() == 2 ? rw.size(0) : 0;
@@ -167,8 +169,9 @@ std::tuple<Tensor, Tensor> sx_router(const Tensor& h, const Tensor& rw, const Op
   TORCH_CHECK(!has(corr) || vec(*corr, at::kFloat, E), "sx_router: correction f32 [E]");
   auto f = h.options().dtype(at::kFloat);
   Tensor idx = at::empty({T, top}, f.dtype(at::kInt)), w = at::empty({T, top}, f);
-  illm::sx::router(bf(h), h.data_ptr(), rw.data_ptr<float>(), has(corr) ? corr->data_ptr<float>() : nullptr, (int)T, (int)W,
-                   (int)E, (int)top, (int)groups, (int)keep, idx.data_ptr<int32_t>(), w.data_ptr<float>(), stream());
+  illm::sx::router(bf(h), h.data_ptr(), rw.data_ptr<float>(), has(corr) ? corr->data_ptr<float>() : nullptr,
+                   {sigmoid, best_two, renorm, (float)scale}, (int)T, (int)W, (int)E,
+                   (int)top, (int)groups, (int)keep, idx.data_ptr<int32_t>(), w.data_ptr<float>(), stream());
   return {idx, w};
 }
 
@@ -328,8 +331,10 @@ TORCH_LIBRARY_FRAGMENT(ipex_llm_amd, m) {
   m.def("sx_add_normed_experts(Tensor(a!) x, Tensor rows, Tensor idx, Tensor wts, Tensor h, int experts, Tensor pa, "
         "Tensor pw, Tensor pb, Tensor? qa, Tensor? qw, Tensor? qb, bool act_f32) -> Tensor");
   m.def("sx_rms_sigmoid_gate(Tensor o, Tensor w, Tensor gate, float eps, bool act_f32) -> Tensor");
-  m.def("sx_route_groups(Tensor z, Tensor? corr, int top, int groups, int keep) -> (Tensor, Tensor)");
-  m.def("sx_router(Tensor h, Tensor rw, Tensor? corr, int top, int groups, int keep) -> (Tensor, Tensor)");
+  m.def("sx_route_groups(Tensor z, Tensor? corr, int top, int groups, int keep, bool sigmoid=False, bool best_two=False, "
+        "bool renorm=False, float scale=1.0) -> (Tensor, Tensor)");
+  m.def("sx_router(Tensor h, Tensor rw, Tensor? corr, int top, int groups, int keep, bool sigmoid=False, bool best_two=False, "
+        "bool renorm=False, float scale=1.0) -> (Tensor, Tensor)");
   m.def("sx_decay_scan(Tensor q, Tensor k, Tensor v, Tensor decay, Tensor(a!) S, Tensor cu, Tensor slots, Tensor pos, "
         "int[] lens, int chunk_min) -> Tensor");
   m.def("sx_delta_scan(Tensor q, Tensor k, Tensor v, Tensor a, Tensor b, Tensor rate, Tensor dt_bias, float q_scale, "

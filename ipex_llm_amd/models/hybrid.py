@@ -70,11 +70,24 @@ Building blocks (each usable by any design that lists it in its layer specs):
   f32 state, multiplied by a tanh-GELU branch.
 * ``ScoredMoE``         experts weighed by their softmax score over *all* router
   outputs, chosen by score + correction inside the best groups; some router
-  outputs may be identity experts (their result is the input itself).
+  outputs may be identity experts (their result is the input itself).  Also
+  with sigmoid scores, groups ranked by their two best, and weights
+  renormalised and scaled (``MoESpec.score`` / ``group`` / ``renorm`` / ``scale``).
+* ``LatentAttention`` also takes a learned sink per head.
+* ``MaskedAttention`` also takes an RMS norm of queries and keys without a weight
+  (``qk_norm="unit"``) and a bias of its output projection.
+* ``ChannelDelta``      the delta rule with one decay per key channel (low-rank),
+  short convolutions with SiLU, per-head RMS norm with a low-rank sigmoid gate.
+* ``TimeMix``           RWKV-6 form of time mixing: receptance, key, value, gate and
+  decay read blends of a token's and its predecessor's input, the state is read
+  before it is written, with a bonus for the current token.
+* ``ScaledSum``         two mixers on the same input, a constant times each result.
 
 Block layouts.  ``pre_norm`` (``PreNormLayer``): x += mixer(norm1(x)),
 x += ff(norm2(x)) with vector RMS norms; each sublayer's result is added by
-the launch that also forms the next norm.  ``post_norm`` (``HybridLayer``): the sublayers read the
+the launch that also forms the next norm; optionally a scale per coordinate on
+every result (``layer_scale``) and norm weights stored around zero
+(``norm = "rms_offset"``).  ``post_norm`` (``HybridLayer``): the sublayers read the
 residual stream ``x`` itself and their *output* is normalised:
 x += mult * LN(mixer(x)), x += mult * LN(ff(x)).  ``parallel``
 (``ParallelLayer``): one norm, both sublayers read it, their scaled results
@@ -89,6 +102,9 @@ input.
 x += N1b(mixer(N1(x))), x += N2b(ff(N2(x))) with statistics-free tanh norms
 (``DynTanh``); a sublayer's result is normed and added, and the next sublayer's
 norm formed, by one launch.
+``HybridSpec.loop``: a range of layers runs several times in a row with the same
+weights, each pass with a cache and state of its own and with
+``x = W_in [x; embedding]`` in front of it.
 The residual stream is f32 throughout; projections run in the model's
 activation dtype through the vendor GEMM, everything else in the kernels of
 ``ops/seqmix.py`` and ``ops/blockmix.py``.
@@ -107,6 +123,7 @@ import torch.nn as nn
 import torch.nn.functional as F
 
 from ..ops import blockmix as BM
+from ..ops import chanmix as CX
 from ..ops import gatedmix as GM
 from ..ops import maskattn as MA
 from ..ops import seqmix as SM
@@ -143,6 +160,7 @@ class LatentAttentionSpec:
     out_gate: bool = True
     gate: str = "head"                      # "head": one gate per head | "element": one per value of the joined heads
     window: int = 0                         # > 0: a token sees itself and the window - 1 tokens before it
+    sink: bool = False                      # a learned number per head in the softmax's denominator
 
 
 @dataclass
@@ -164,8 +182,10 @@ class MaskedAttentionSpec:
     scale: float
     rot: Optional[RotarySpec] = None        # on the first rot.dims values of every head
     mask: MaskSpec = None
-    qk_norm: str = "whole"                  # "none" | "head" (weights [dim]) | "whole" (weights [heads dim])
+    qk_norm: str = "whole"                  # "none" | "head" (weights [dim]) | "whole" (weights [heads dim]) | "unit" (per
+                                            # head, no weight; a plain rotation commutes with it)
     bias: bool = True                       # q / k / v projections carry biases
+    out_bias: bool = False                  # so does the output projection
     sink: bool = True                       # a learned number per head in the softmax's denominator
     kv_from: Optional[int] = None           # read this layer's cache rows instead of projecting keys and values
     taps: int = 0                           # >= 1: causal per-channel convolutions on q / k / v right after the projection
@@ -214,6 +234,34 @@ class RealGatedLRUSpec:
     blocks: int                             # of the block-diagonal gate matrices
     taps: int
     power: float = 8.0                      # log a = -power r softplus(lam)
+
+
+@dataclass
+class ChannelDeltaSpec:
+    heads: int
+    kv_heads: int                           # query / key heads; head h reads h // (heads / kv_heads)
+    dim: int
+    vdim: int
+    taps: int                               # of the convolutions on q / k / v
+    rank: int                               # of the decay's low-rank projection
+    gate_rank: int                          # of the output gate's
+
+
+@dataclass
+class TimeMixSpec:
+    heads: int
+    dim: int                                # key and value size per head
+    rank: int                               # of the decay's low-rank projection
+
+
+@dataclass
+class ScaledSumSpec:
+    left: object                            # specs of MIXERS
+    right: object
+    left_scale: float
+    right_scale: float
+    left_kind: str = "masked_attention"
+    right_kind: str = "time_mix"
 
 
 @dataclass
@@ -273,6 +321,10 @@ class MoESpec:
     identity: int = 0                       # the last router outputs beyond ``experts``: their result is the input
     groups: int = 1                         # equal groups of neighbouring router outputs ...
     keep: int = 1                           # ... of which the best ones take part in the choice
+    score: str = "softmax"                  # or "sigmoid"
+    group: str = "max"                      # a group's score: its largest corrected score, or "top2": the two largest's sum
+    renorm: bool = False                    # the winners' weights over their sum, times ``scale``
+    scale: float = 1.0
 
 
 @dataclass
@@ -290,6 +342,13 @@ class BigramSpec:
 
 
 @dataclass
+class LoopSpec:
+    start: int                              # layers start .. stop - 1 run ``times`` times in a row
+    stop: int
+    times: int
+
+
+@dataclass
 class HybridSpec:
     model_type: str
     vocab_size: int
@@ -302,10 +361,12 @@ class HybridSpec:
     logit_scale: float = 1.0                # the logits are multiplied by it
     block: str = "post_norm"                # "post_norm" | "parallel" | "parallel2" | "pre_norm" | "sandwich"
     norm: str = "layer_norm"                # "layer_norm" | "rms_scalar" (one number) | "rms" (a vector) | "dyn_tanh"
-    layer_scale: bool = False               # parallel blocks: per-coordinate scales on both sublayers' results
+                                            # | "rms_offset" (a vector stored around zero: times 1 + w)
+    layer_scale: bool = False               # per-coordinate scales on both sublayers' results
     canon_taps: int = 0                     # parallel blocks: taps of the convolution in front of the mixer (0: none)
     side_dim: int = 0                       # per-layer slice of the token-side table (0: none)
     tied_head: bool = False                 # the logits are products with the embedding table
+    loop: Optional[LoopSpec] = None         # pre_norm blocks
 
     @property
     def num_layers(self) -> int:
@@ -321,7 +382,7 @@ def _spec_list(c) -> list:
 class LatentAttention(nn.Module):
     cache_kind = "rows"
 
-    def __init__(self, s: LatentAttentionSpec, w_q, w_dkv, dkv_norm, w_uk, w_uv, w_g, w_o):
+    def __init__(self, s: LatentAttentionSpec, w_q, w_dkv, dkv_norm, w_uk, w_uv, w_g, w_o, sink=None):
         super().__init__()
         self.s = s
         H, r = s.heads, s.kv_rank
@@ -343,6 +404,7 @@ class LatentAttention(nn.Module):
         self.dkv_norm = nn.Parameter(dkv_norm, requires_grad=False)
         self.w_uk = nn.Parameter(w_uk.view(H, s.dim, r).contiguous(), requires_grad=False)               # [H, dim, r]
         self.w_uv_t = nn.Parameter(w_uv.view(H, s.vdim, r).transpose(1, 2).contiguous(), requires_grad=False)  # [H, r, dv]
+        self.sink = nn.Parameter(sink.float().contiguous(), requires_grad=False) if s.sink else None
         self.w_o = nn.Parameter(w_o, requires_grad=False)
         self.table: Optional[torch.Tensor] = None
 
@@ -358,7 +420,7 @@ class LatentAttention(nn.Module):
     def forward(self, xa, pos, slots, meta: AttnMeta, cache, li: int, eps: float):
         s = self.s
         T, H = xa.shape[0], s.heads
-        y = F.linear(xa, self.w_in)
+        y = BM.linear(xa, self.w_in)
         q = y[:, :self.n_q].reshape(T, H, s.dim + s.rot_dim).contiguous()
         dkv = y[:, self.n_q:self.n_q + self.n_dkv]
         gate = y[:, self.n_q + self.n_dkv:] if s.out_gate else None
@@ -370,7 +432,7 @@ class LatentAttention(nn.Module):
         q_lat = torch.bmm(q[..., :s.dim].transpose(0, 1), self.w_uk).transpose(0, 1)
         o_lat = SM.latent_attention(q_lat, q[..., s.dim:], cache.rows[li], meta.block_tables, meta.seq_of, pos,
                                     s.scale, head_gate, meta.q_lens_host, meta.seq_lens_host, xa.dtype,
-                                    window=s.window)
+                                    window=s.window, sink=self.sink)
         o = torch.bmm(o_lat.transpose(0, 1), self.w_uv_t).transpose(0, 1).reshape(T, H * s.vdim)
         if gate is not None and s.gate == "element":
             o = MA.sigmoid_gate(o, gate)
@@ -488,7 +550,7 @@ class MaskedAttention(nn.Module):
     cache_kind = "rows"
 
     def __init__(self, s: MaskedAttentionSpec, w_q, w_k, w_v, b_q, b_k, b_v, q_norm, k_norm, sink, w_o, conv=None,
-                 talk=None, w_g=None, temp=None):
+                 talk=None, w_g=None, temp=None, b_o=None):
         super().__init__()
         if s.heads % s.kv_heads:
             raise ValueError("heads must be a multiple of kv_heads")
@@ -496,8 +558,12 @@ class MaskedAttention(nn.Module):
             raise ValueError("mask: causal, or window / chunk with a size of at least 1")
         if s.mask.keep_first and s.mask.kind != "window":
             raise ValueError("keep_first belongs to a window")
-        if s.qk_norm not in ("none", "head", "whole"):
+        if s.qk_norm not in ("none", "head", "whole", "unit"):
             raise ValueError(f"unknown qk_norm {s.qk_norm!r}")
+        if s.qk_norm == "unit":                 # a rotation without a magnitude leaves the mean square as it is
+            if s.rot is not None and s.rot.scaling and "low" not in s.rot.scaling:
+                raise ValueError("qk_norm 'unit' needs a rotation that keeps lengths (no YaRN scaling)")
+            q_norm = k_norm = torch.ones(s.dim, dtype=w_q.dtype, device=w_q.device)
         if s.out_gate and s.gate not in ("head", "element"):
             raise ValueError(f"unknown gate kind {s.gate!r}")
         self.s = s
@@ -525,6 +591,7 @@ class MaskedAttention(nn.Module):
         self.talk = nn.Parameter(talk.float().contiguous(), requires_grad=False) if s.talk else None
         self.temp = nn.Parameter(temp.float().contiguous(), requires_grad=False) if s.temp else None
         self.w_o = nn.Parameter(w_o, requires_grad=False)
+        self.b_o = nn.Parameter(b_o.contiguous(), requires_grad=False) if s.out_bias else None
         self.table: Optional[torch.Tensor] = None
 
     def cache_spec(self):
@@ -572,7 +639,7 @@ class MaskedAttention(nn.Module):
                                 keep_first=s.mask.keep_first, talk=self.talk)
         if gate is not None:
             o = MA.sigmoid_gate(o, gate)
-        return BM.linear(o, self.w_o)
+        return BM.linear(o, self.w_o, self.b_o)
 
 
 class MinGRU(nn.Module):
@@ -819,6 +886,176 @@ class SideBySide(nn.Module):
         return GM.rms_pair_mean(p.a, p.b, p.wa, p.wb, eps, xa.dtype)
 
 
+class ChannelDelta(nn.Module):
+    """``w_q`` / ``w_k`` [K d, W], ``w_v`` [H dv, W], ``w_b`` [H, W], ``w_a1`` [rank, W], ``w_a2`` [H d, rank],
+    ``w_g1`` [gate_rank, W], ``w_g2`` [H dv, gate_rank], ``conv`` = (q, k, v) weights [channels, taps], ``a_log`` [H],
+    ``dt_bias`` [H d], ``norm`` [dv], ``w_o`` [W, H dv]."""
+    cache_kind = "state"
+
+    def __init__(self, s: ChannelDeltaSpec, w_q, w_k, w_v, w_b, w_a1, w_a2, w_g1, w_g2, conv, a_log, dt_bias, norm, w_o):
+        super().__init__()
+        if s.heads % s.kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        if s.taps < 1 or s.taps > 16:
+            raise ValueError("1 <= conv taps <= 16")
+        self.s = s
+        self.n_qkv = int(w_q.shape[0] + w_k.shape[0] + w_v.shape[0])
+        self.w_in = nn.Parameter(torch.cat([w_q, w_k, w_v, w_b, w_a1, w_g1], 0).contiguous(), requires_grad=False)
+        self.b_in = None
+        self.conv = nn.Parameter(torch.cat(list(conv), 0).float().contiguous(), requires_grad=False)
+        self.rate = nn.Parameter(a_log.double().exp().float().repeat_interleave(s.dim).contiguous(), requires_grad=False)
+        self.dt_bias = nn.Parameter(dt_bias.float().contiguous(), requires_grad=False)
+        self.w_a2 = nn.Parameter(w_a2.contiguous(), requires_grad=False)
+        self.w_g2 = nn.Parameter(w_g2.contiguous(), requires_grad=False)
+        self.norm = nn.Parameter(norm.repeat(s.heads).contiguous(), requires_grad=False)        # shared by the heads
+        self.w_o = nn.Parameter(w_o, requires_grad=False)
+
+    def cache_spec(self):
+        s = self.s
+        return ("state", {"chan_delta": (s.heads, s.dim, s.vdim), "conv": (s.taps - 1, self.n_qkv)})
+
+    def ensure_table(self, max_pos: int):
+        return None
+
+    def forward(self, xa, pos, slots, meta: AttnMeta, cache, li: int, eps: float):
+        return self.mix(BM.linear(xa, self.w_in), pos, slots, meta, cache, li, eps)
+
+    def mix(self, y, pos, slots, meta: AttnMeta, cache, li: int, eps: float):
+        s, st = self.s, cache.state[li]
+        T, H, K, d, dv = y.shape[0], s.heads, s.kv_heads, s.dim, s.vdim
+        n = self.n_qkv
+        b, a1, g1 = y[:, n:n + H], y[:, n + H:n + H + s.rank], y[:, n + H + s.rank:]
+        u = SSM.conv_silu(y[:, :n], self.conv, None, st["conv"], meta.cu_q, meta.seq_of, meta.state_slots, pos,
+                          meta.q_lens_host)
+        q, k, v = u[:, :K * d].view(T, K, d), u[:, K * d:2 * K * d].view(T, K, d), u[:, 2 * K * d:].view(T, H, dv)
+        g = CX.lowrank_decay(a1, self.w_a2, self.rate, self.dt_bias, "softplus").view(T, H, d)
+        o = CX.channel_delta_scan(q, k, v, g, b, d ** -0.5, st["chan_delta"], meta.cu_q, meta.state_slots, pos,
+                                  meta.q_lens_host)
+        gate = BM.linear(g1.contiguous(), self.w_g2)
+        return BM.linear(SM.head_rms_gate(o, self.norm, gate, eps, y.dtype), self.w_o)
+
+
+class TimeMix(nn.Module):
+    """``mu`` f32 [5, W] (of r, k, v, g, w), ``w_rkvg`` four matrices [H d, W], ``w_w1`` [rank, W], ``w_w2`` [H d, rank],
+    ``w0`` [H d], ``u`` [H, d], ``norm`` [H d], ``w_o`` [W, H d]."""
+    cache_kind = "state"
+
+    def __init__(self, s: TimeMixSpec, mu, w_rkvg, w_w1, w_w2, w0, u, norm, w_o):
+        super().__init__()
+        self.s = s
+        n = s.heads * s.dim
+        self.sizes = [n] * 4 + [int(w_w1.shape[0])]
+        # every row group reads a blend of its own: decode steps run all of them as one launch over ``w_in``, longer
+        # steps the four equal ones as a batched product over ``w_t`` [4, W, H d]
+        self.w_in = nn.Parameter(torch.cat([*w_rkvg, w_w1], 0).contiguous(), requires_grad=False)
+        self.b_in = None
+        self.w_t = nn.Parameter(torch.stack([w.t() for w in w_rkvg]).contiguous(), requires_grad=False)
+        self.mu = nn.Parameter(mu.float().contiguous(), requires_grad=False)
+        self.w_w2 = nn.Parameter(w_w2.contiguous(), requires_grad=False)
+        self.w0 = nn.Parameter(w0.float().contiguous(), requires_grad=False)
+        self.u = nn.Parameter(u.float().reshape(s.heads, s.dim).contiguous(), requires_grad=False)
+        self.norm = nn.Parameter(norm.contiguous(), requires_grad=False)
+        self.w_o = nn.Parameter(w_o, requires_grad=False)
+
+    def cache_spec(self):
+        s = self.s
+        return ("state", {"time_mix": (s.heads, s.dim, s.dim), "time_mix_shift": (self.mu.shape[1],)})
+
+    def ensure_table(self, max_pos: int):
+        return None
+
+    def mixes(self, xa, pos, meta: AttnMeta, cache, li: int):
+        return CX.token_mixes(xa, self.mu, cache.state[li]["time_mix_shift"], meta.cu_q, meta.seq_of, meta.state_slots,
+                              pos, meta.q_lens_host)
+
+    def project(self, m):
+        """blends [5, T, W] -> r, k, v, g [T, H d] each, the decay's [T, rank]"""
+        n = self.sizes[0]
+        w1 = self.w_in[4 * n:]
+        p = torch.bmm(m[:4], self.w_t)
+        return p[0], p[1], p[2], p[3], BM.linear(m[4], w1)
+
+    def forward(self, xa, pos, slots, meta: AttnMeta, cache, li: int, eps: float):
+        m = self.mixes(xa, pos, meta, cache, li)
+        if CX.grouped_fits(xa.shape[0], self.w_in):
+            parts = CX.grouped_linear(list(m.unbind(0)), self.sizes, self.w_in).split(self.sizes, 1)
+        else:
+            parts = self.project(m)
+        return self.mix(parts, pos, slots, meta, cache, li, eps)
+
+    def mix(self, parts, pos, slots, meta: AttnMeta, cache, li: int, eps: float):
+        s = self.s
+        r, k, v, g, a = parts
+        T, H, d = r.shape[0], s.heads, s.dim
+        w = CX.lowrank_decay(a, self.w_w2, None, self.w0, "exp", squash=True).view(T, H, d)
+        o = CX.bonus_scan(r.view(T, H, d), k.view(T, H, d), v.view(T, H, d), w, self.u, cache.state[li]["time_mix"],
+                          meta.cu_q, meta.state_slots, pos, meta.q_lens_host)
+        return BM.linear(SM.head_rms_gate(o, self.norm, g, eps, r.dtype, silu=True), self.w_o)
+
+
+class ScaledSum(nn.Module):
+    """Two mixers reading the same input: ``left_scale * left + right_scale * right``.  ``left`` reads one projection of
+    the input (``w_in`` / ``mix``), ``right`` is a ``TimeMix``: decode steps run both mixers' projections as one launch
+    over row groups."""
+    cache_kind = "both"
+
+    def __init__(self, left: nn.Module, right: TimeMix, left_scale: float, right_scale: float, width: int):
+        super().__init__()
+        self.left, self.right = left, right
+        self.scales = (float(left_scale), float(right_scale))
+        self.n_left = int(left.w_in.shape[0])
+        self.w_in = nn.Parameter(torch.cat([left.w_in.data, right.w_in.data], 0).contiguous(), requires_grad=False)
+        self.b_in = None
+        if left.b_in is not None:
+            b = left.b_in.data
+            self.b_in = nn.Parameter(torch.cat([b, torch.zeros(right.w_in.shape[0], dtype=b.dtype, device=b.device)])
+                                     .contiguous(), requires_grad=False)
+        right.w_in.data = self.w_in.data[self.n_left:]       # one copy: both mixers' rows are parts of it
+        left.w_in = left.b_in = None
+        dev = self.w_in.device
+        self.register_buffer("one", torch.ones(width, dtype=torch.float32, device=dev), persistent=False)
+
+    def cache_spec(self):
+        return [c for m in (self.left, self.right) for c in _spec_list(m.cache_spec()) if c is not None]
+
+    def ensure_table(self, max_pos: int):
+        self.left.ensure_table(max_pos)
+
+    @property
+    def table(self):
+        return getattr(self.left, "table", None)
+
+    @table.setter
+    def table(self, v):
+        self.left.table = v
+
+    def parts(self, xa, pos, slots, meta: AttnMeta, cache, li: int, eps: float, scale: Optional[torch.Tensor] = None):
+        """both mixers' results, their scaled sum (times ``scale`` [W]) still to be formed"""
+        m = self.right.mixes(xa, pos, meta, cache, li)
+        n = self.n_left
+        if CX.grouped_fits(xa.shape[0], self.w_in):
+            y = CX.grouped_linear([xa, *m.unbind(0)], [n, *self.right.sizes], self.w_in, self.b_in)
+            yl, parts = y[:, :n], y[:, n:].split(self.right.sizes, 1)
+        else:
+            yl = BM.linear(xa, self.w_in[:n], self.b_in[:n] if self.b_in is not None else None)
+            parts = self.right.project(m)
+        a = self.left.mix(yl, pos, slots, meta, cache, li, eps)
+        b = self.right.mix(parts, pos, slots, meta, cache, li, eps)
+        s = self.one if scale is None else scale
+        sa, sb = self._scaled(s)
+        return CX.Pending(a, sa, b, sb)
+
+    def _scaled(self, s: torch.Tensor):
+        """``s`` times both constants (kept: the same layer scale comes every step)"""
+        c = getattr(self, "_cached", None)
+        if c is None or c[0] is not s or c[1].device != s.device:
+            c = self._cached = (s, s.detach() * self.scales[0], s.detach() * self.scales[1])
+        return c[1], c[2]
+
+    def forward(self, xa, pos, slots, meta: AttnMeta, cache, li: int, eps: float):
+        return self.parts(xa, pos, slots, meta, cache, li, eps).value().to(xa.dtype)
+
+
 class GroupedAttention(nn.Module):
     cache_kind = "rows"
 
@@ -915,8 +1152,8 @@ class SoftmaxMoE(nn.Module):
 class ScoredMoE(nn.Module):
     """``router`` [experts + identity, W], ``correction`` [experts + identity] or None, ``w_gu`` [E, 2 ff, W] (every
     expert's gate rows, then its up rows), ``w_down`` [E, W, ff].  Scores are the softmax of f32 logits over all router
-    outputs; the choice goes by score + correction inside the best groups, the weights are the plain scores and
-    multiply the experts' *outputs*; experts ``W_down (silu(W_gate h) * (W_up h))``, identity experts ``h``."""
+    outputs, or their sigmoids; the choice goes by score + correction inside the best groups, the weights are the plain
+    scores, or renormalised and scaled, and multiply the experts' *outputs*; experts ``W_down (silu(W_gate h) * (W_up h))``, identity experts ``h``."""
 
     def __init__(self, s: MoESpec, router, correction, w_gu, w_down):
         super().__init__()
@@ -928,11 +1165,12 @@ class ScoredMoE(nn.Module):
         self.correction = nn.Parameter(correction.float().contiguous(), requires_grad=False) if correction is not None else None
         self.w_gu = nn.Parameter(w_gu.contiguous(), requires_grad=False)
         self.w_down = nn.Parameter(w_down.contiguous(), requires_grad=False)
+        self.rule = SX.RouteRule(s.score, s.group, s.renorm, s.scale)
 
     def parts(self, xa) -> SX.ExpertSum:
         """the chosen experts' weighted results, their sum still to be formed"""
         s = self.s
-        idx, wts = SX.route(xa, self.router, self.correction, s.top, s.groups, s.keep)
+        idx, wts = SX.route(xa, self.router, self.correction, s.top, s.groups, s.keep, self.rule)
         rows = BM.moe_expert_rows(xa, idx, wts, self.w_gu, self.w_down, float("inf"), 1.0, 0.0, "output", s.identity)
         return SX.ExpertSum(rows, idx, wts, xa, s.experts)
 
@@ -976,27 +1214,49 @@ class HybridLayer(nn.Module):
 
 
 class PreNormLayer(nn.Module):
-    """x += mixer(norm1(x)); x += ff(norm2(x)).  ``carry`` is the previous sublayer's result that is not yet in
+    """x += mixer(norm1(x)); x += ff(norm2(x)); with ``ls1`` / ``ls2`` [W] every result times its scale, and then the norms'
+    weights are f32 and the results travel as ``Pending``.  ``carry`` is the previous sublayer's result that is not yet in
     ``x`` (None at the first layer): the launch that forms a norm adds it first, and the layer hands its own last
     result on the same way (the model adds the final one with its own norm)."""
 
-    def __init__(self, mixer: nn.Module, norm1: torch.Tensor, mlp: Optional[nn.Module], norm2: Optional[torch.Tensor]):
+    def __init__(self, mixer: nn.Module, norm1: torch.Tensor, mlp: Optional[nn.Module], norm2: Optional[torch.Tensor],
+                 ls1: Optional[torch.Tensor] = None, ls2: Optional[torch.Tensor] = None):
         super().__init__()
         self.mixer, self.mlp = mixer, mlp
         self.norm1 = nn.Parameter(norm1, requires_grad=False)
         self.norm2 = nn.Parameter(norm2, requires_grad=False) if norm2 is not None else None
+        self.ls1 = nn.Parameter(ls1.float().contiguous(), requires_grad=False) if ls1 is not None else None
+        self.ls2 = nn.Parameter(ls2.float().contiguous(), requires_grad=False) if ls2 is not None else None
+        if ls1 is not None and isinstance(mixer, ScaledSum):
+            mixer._scaled(self.ls1)
 
     def cache_specs(self):
         return _spec_list(self.mixer.cache_spec())
 
     def forward(self, x, carry, ids, pos, slots, meta, cache, li: int, model):
         s, act = model.spec, model.dtype
+        if self.ls1 is not None:
+            return self._scaled(x, carry, pos, slots, meta, cache, li, s.norm_eps, act)
         h = BM.add_rms_norm_rows_(x, carry, self.norm1, s.norm_eps, act)
         y = self.mixer(h, pos, slots, meta, cache, li, s.norm_eps)
         if self.mlp is None:
             return y
         h = BM.add_rms_norm_rows_(x, y, self.norm2, s.norm_eps, act)
         return self.mlp(h)
+
+    def _scaled(self, x, carry, pos, slots, meta, cache, li: int, eps: float, act) -> CX.Pending:
+        h = CX.add_scaled_norm_(x, carry, self.norm1, eps, act)
+        if isinstance(self.mixer, ScaledSum):
+            y = self.mixer.parts(h, pos, slots, meta, cache, li, eps, self.ls1)
+        else:
+            y = CX.Pending(self.mixer(h, pos, slots, meta, cache, li, eps), self.ls1)
+        if self.mlp is None:
+            return y
+        h = CX.add_scaled_norm_(x, y, self.norm2, eps, act)
+        if isinstance(self.mlp, ScoredMoE) and not self.mlp.s.identity:
+            return CX.Pending(self.mlp.parts(h).rows, self.ls2)
+        y = self.mlp(h)
+        return CX.Pending(y[0] if isinstance(y, tuple) else y, self.ls2)
 
 
 class ParallelLayer(nn.Module):
@@ -1118,6 +1378,8 @@ MIXERS: Dict[str, tuple] = {"latent_attention": (LatentAttentionSpec, LatentAtte
                             "lightning": (LightningSpec, LightningAttention),
                             "gated_delta": (GatedDeltaSpec, GatedDelta),
                             "real_gated_lru": (RealGatedLRUSpec, RealGatedLRU),
+                            "channel_delta": (ChannelDeltaSpec, ChannelDelta), "time_mix": (TimeMixSpec, TimeMix),
+                            "scaled_sum": (ScaledSumSpec, ScaledSum),
                             "side_by_side": (SideBySideSpec, SideBySide)}
 
 
@@ -1128,9 +1390,11 @@ class HybridCausalLM(nn.Module):
 
     def __init__(self, spec: HybridSpec, embed: torch.Tensor, bigram: Optional[torch.Tensor],
                  layers: List[nn.Module], final_norm, head: Optional[torch.Tensor], dtype=torch.bfloat16,
-                 side_embed: Optional[torch.Tensor] = None):
+                 side_embed: Optional[torch.Tensor] = None, loop_in: Optional[torch.Tensor] = None):
         super().__init__()
         self.spec, self.dtype = spec, dtype
+        self.loop_in = nn.Parameter(loop_in, requires_grad=False) if loop_in is not None else None
+        self.runs = self._runs(spec, len(layers))
         self.embed_tokens = nn.Parameter(embed, requires_grad=False)
         self.bigram = nn.Parameter(bigram, requires_grad=False) if bigram is not None else None
         self.side_embed = nn.Parameter(side_embed, requires_grad=False) if side_embed is not None else None
@@ -1142,9 +1406,25 @@ class HybridCausalLM(nn.Module):
         self.first_stage = self.last_stage = True
         self.capture_layers: Optional[list] = None      # debugging: residual stream after every layer
 
+    @staticmethod
+    def _runs(spec: HybridSpec, n: int):
+        """the layers in the order they run, as (layer, first of a loop's pass); every run has a cache entry of its own"""
+        lp = spec.loop
+        if lp is None:
+            return [(i, False) for i in range(n)]
+        if spec.block != "pre_norm" or not 0 <= lp.start < lp.stop <= n or lp.times < 1:
+            raise ValueError("a loop needs pre-norm blocks, 0 <= start < stop <= layers and times >= 1")
+        if any(getattr(L.mixer, "kv_from", None) is not None for L in spec.layers):
+            raise ValueError("a loop's passes have caches of their own: no layer may read another one's rows")
+        body = [(i, i == lp.start) for i in range(lp.start, lp.stop)] * lp.times
+        return [(i, False) for i in range(lp.start)] + body + [(i, False) for i in range(lp.stop, n)]
+
     @property
     def device(self):
         return self.embed_tokens.device
+
+    def _cache_specs(self) -> list:
+        return [self.layers[i].cache_specs() for i, _ in self.runs]
 
     @property
     def has_state(self) -> bool:
@@ -1159,7 +1439,7 @@ class HybridCausalLM(nn.Module):
 
     def cache_bytes_per_token(self) -> int:
         eb = torch.empty(0, dtype=self.dtype).element_size()
-        return sum(c[1] * eb for L in self.layers for c in L.cache_specs() if c is not None and c[0] == "rows")
+        return sum(c[1] * eb for run in self._cache_specs() for c in run if c is not None and c[0] == "rows")
 
     def make_cache(self, max_tokens: int, batch: int = 1, block_size: int = 64, kv_fp8: int = 0,
                    num_blocks: Optional[int] = None, num_slots: Optional[int] = None):
@@ -1168,7 +1448,7 @@ class HybridCausalLM(nn.Module):
             raise ValueError("hybrid decoders keep their latent rows in the activation dtype (no fp8 cache)")
         nblk = num_blocks or batch * ((max_tokens + block_size - 1) // block_size)
         self.ensure_rope_cache(max_tokens + 1)
-        return HybridCache([L.cache_specs() for L in self.layers], nblk, num_slots or batch, block_size,
+        return HybridCache(self._cache_specs(), nblk, num_slots or batch, block_size,
                            self.dtype, self.device)
 
     @staticmethod
@@ -1211,17 +1491,26 @@ class HybridCausalLM(nn.Module):
             xa = SX.dyn_tanh(x, (self.layers[0].pre1 if len(self.layers) else self.norm).args, act)
         else:
             xa = None if pre else (x if act == torch.float32 else x.to(act))
-        for li, L in enumerate(self.layers):
-            xa = L(x, xa, ids, pos, slots, meta, cache, li, self)
+        def pending(y):                     # a pre-norm layer's result as f32 rows
+            return y.value() if isinstance(y, CX.Pending) else y.float()
+        for li, (i, first) in enumerate(self.runs):
+            if first:                       # x = W_in [x; embedding] in front of a loop's pass
+                if xa is not None and not isinstance(xa, CX.Pending):
+                    x, xa = x.add_(xa.float()), None
+                x, xa = CX.linear_f32(CX.loop_input(x, xa, self.embed_tokens, ids), self.loop_in), None
+            xa = self.layers[i](x, xa, ids, pos, slots, meta, cache, li, self)
             if self.capture_layers is not None:
-                self.capture_layers.append(x + xa.float() if pre else x.clone())
+                self.capture_layers.append(x + pending(xa) if pre else x.clone())
         if not self.last_stage:
-            return x.add_(xa.float()) if pre and xa is not None else x
+            return x.add_(pending(xa)) if pre and xa is not None else x
         if logits_idx is not None:
             x = x.index_select(0, logits_idx)
-            xa = xa.index_select(0, logits_idx) if xa is not None else xa
+            if xa is not None:
+                xa = xa.select(logits_idx) if isinstance(xa, CX.Pending) else xa.index_select(0, logits_idx)
         if s.block == "sandwich":
             xn = xa                         # the last layer formed the final norm
+        elif pre and s.norm == "rms_offset":
+            xn = CX.add_scaled_norm_(x, xa, self.norm, s.norm_eps, act)
         elif pre:
             xn = BM.add_rms_norm_rows_(x, xa, self.norm, s.norm_eps, act)
         elif s.norm == "layer_norm":

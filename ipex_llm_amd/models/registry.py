@@ -21,6 +21,7 @@ NATIVE_ARCHITECTURES = {
     "Vogolix": "ipex_llm_amd.models.vogolix",
     "Zoguzen": "ipex_llm_amd.models.zoguzen",
     "Sudosun": "ipex_llm_amd.models.sudosun",
+    "Lokolorn": "ipex_llm_amd.models.lokolorn",
 }
 
 

@@ -74,7 +74,7 @@ def require_seqmix():
     if full:
         lib = require()
         if not hasattr(lib, "sm_latent_attention") or not hasattr(lib, "bm_talk_attention") or \
-                not hasattr(lib, "sx_delta_scan"):
+                not hasattr(lib, "sx_delta_scan") or not hasattr(lib, "cx_delta_scan"):
             raise RuntimeError(f"{_LIB_PATH} predates the sequence-mixing kernels: rebuild it "
                                "(python -m ipex_llm_amd._build)")
         return lib

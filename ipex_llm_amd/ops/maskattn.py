@@ -112,6 +112,8 @@ GEMM_MIN_CHUNK = int(os.environ.get("ILLM_MASKATTN_GEMM_MIN", "128"))
 # queries: a block's keys are the kept first tokens and everything from its first query's window start on.
 WINDOW_GEMM_MIN = int(os.environ.get("ILLM_MASKATTN_WINDOW_GEMM_MIN", "1536"))
 WINDOW_Q_BLOCK = int(os.environ.get("ILLM_MASKATTN_WINDOW_BLOCK", "512"))
+# The same with the whole past visible (a window as long as the context).
+CAUSAL_GEMM_MIN = int(os.environ.get("ILLM_MASKATTN_CAUSAL_GEMM_MIN", "512"))
 
 
 def masked_attention(q: torch.Tensor, rows: torch.Tensor, G: int, dv: int, block_tables: torch.Tensor,
@@ -261,15 +263,16 @@ def _masked_attention_gpu(q, rows, G, dv, block_tables, seq_of, pos, scale, mask
     code = MASKS[mask]
     big = mask == "chunk" and GEMM_MIN_CHUNK > 0 and max(q_lens) >= GEMM_MIN_CHUNK and _bmm_f32_ok(rows.dtype) and \
         (talk is None or H <= 256)
-    if mask == "window" and WINDOW_GEMM_MIN > 0 and max(q_lens) >= WINDOW_GEMM_MIN and _bmm_f32_ok(rows.dtype) and \
-            (talk is None or H <= 256):
+    min_q = {"window": WINDOW_GEMM_MIN, "causal": CAUSAL_GEMM_MIN}.get(mask, 0)
+    if min_q > 0 and max(q_lens) >= min_q and _bmm_f32_ok(rows.dtype) and (talk is None or H <= 256):
         # long portions run block by block as library products, the others (decoded tokens, short portions) together
         # through the one-pass kernel
         out = torch.empty(T, H * dv, dtype=out_dtype, device=q.device)
         rest, rest_ctx, t0 = [], 1, 0
         for b, (n, L) in enumerate(zip(q_lens, ctx_lens)):
-            if n >= WINDOW_GEMM_MIN:
-                _window_gemm(q, rows, block_tables[b], G, dv, scale, sink, t0, n, L, size, keep_first, out, softcap, talk)
+            if n >= min_q:
+                _window_gemm(q, rows, block_tables[b], G, dv, scale, sink, t0, n, L, size if mask == "window" else L,
+                             keep_first if mask == "window" else 0, out, softcap, talk)
             elif n:
                 rest.append(torch.arange(t0, t0 + n, device=q.device))
                 rest_ctx = max(rest_ctx, L)

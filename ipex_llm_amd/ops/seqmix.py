@@ -157,7 +157,8 @@ def latent_kv_store(dkv: torch.Tensor, norm_w: torch.Tensor, eps: float, rank: i
 # ------------------------------------------------------------------ latent attention
 def latent_attention(q_lat: torch.Tensor, q_rot: torch.Tensor, rows: torch.Tensor, block_tables: torch.Tensor,
                      seq_of: torch.Tensor, pos: torch.Tensor, scale: float, gate: Optional[torch.Tensor],
-                     q_lens: List[int], ctx_lens: List[int], out_dtype: torch.dtype, window: int = 0) -> torch.Tensor:
+                     q_lens: List[int], ctx_lens: List[int], out_dtype: torch.dtype, window: int = 0,
+                     sink: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Causal softmax attention in the latent space over the paged rows
     ``[latent (r) | rotated key (dr)]``: for token t of sequence b and head h
 
@@ -166,13 +167,14 @@ def latent_attention(q_lat: torch.Tensor, q_rot: torch.Tensor, rows: torch.Tenso
 
     (scores, softmax and the weighted sum in f32).  ``window`` > 0: only the
     keys pos[t] - window < j <= pos[t] count (the token itself and the
-    window - 1 before it).  ``q_rot`` may be a strided view.  ``q_lens`` /
+    window - 1 before it).  ``sink`` f32 [H]: one more term exp(sink[h]) of head
+    h's denominator, without a key or a value.  ``q_rot`` may be a strided view.  ``q_lens`` /
     ``ctx_lens``: host copies of every sequence's new-token count and key count."""
     T, H, r = q_lat.shape
     window = int(window or 0)
     if native(q_lat):
         return _latent_attention_gpu(q_lat, q_rot, rows, block_tables, seq_of, pos, float(scale), gate, q_lens,
-                                     ctx_lens, out_dtype, window)
+                                     ctx_lens, out_dtype, window, sink)
     out = torch.empty(T, H, r, dtype=torch.float32, device=q_lat.device)
     bs = rows.shape[1]
     t0 = 0
@@ -187,7 +189,9 @@ def latent_attention(q_lat: torch.Tensor, q_rot: torch.Tensor, rows: torch.Tenso
         j, p = torch.arange(L, device=sc.device)[None, :], pos[t0:t0 + n].long()[:, None]
         vis = (j <= p) & (j > p - window) if window > 0 else j <= p
         sc = sc.masked_fill(~vis[:, None, :], float("-inf"))
-        out[t0:t0 + n] = torch.einsum("thl,lr->thr", torch.softmax(sc, -1), c)
+        if sink is not None:                                         # one more column, dropped after the softmax
+            sc = torch.cat([sc, sink.float()[None, :, None].expand(n, H, 1)], -1)
+        out[t0:t0 + n] = torch.einsum("thl,lr->thr", torch.softmax(sc, -1)[..., :L], c)
         t0 += n
     if gate is not None:
         out = out * torch.sigmoid(gate.float())[..., None]
@@ -221,7 +225,8 @@ def _mm_f32(a: torch.Tensor, b: torch.Tensor) -> torch.Tensor:
     return a.float() @ b.float()
 
 
-def _latent_attention_gemm(q_lat, q_rot, rows, table_row, pos, scale, L: int, n: int, window: int = 0) -> torch.Tensor:
+def _latent_attention_gemm(q_lat, q_rot, rows, table_row, pos, scale, L: int, n: int, window: int = 0,
+                           sink=None) -> torch.Tensor:
     """one sequence's portion of n >= GEMM_MIN_Q tokens ending at key count L -> f32 [n, H, r]"""
     _, H, r = q_lat.shape
     bs = rows.shape[1]
@@ -235,7 +240,7 @@ def _latent_attention_gemm(q_lat, q_rot, rows, table_row, pos, scale, L: int, n:
         k0 = max(0, L - n + t0 - window + 1) // 8 * 8 if window > 0 else 0      # the first key its first token sees
         q2 = torch.cat([q_lat[t0:t1], q_rot[t0:t1]], -1).reshape((t1 - t0) * H, -1)
         sc = _mm_f32(q2, kv[k0:Lb].t()).contiguous()
-        hi, lo = _ops().sm_causal_softmax(sc, pos[t0:t1].contiguous(), H, scale, f32, k0, window)
+        hi, lo = _ops().sm_causal_softmax(sc, pos[t0:t1].contiguous(), H, scale, f32, k0, window, sink)
         c = kv[k0:Lb, :r]
         o = _mm_f32(hi, c)
         if not f32:
@@ -245,7 +250,7 @@ def _latent_attention_gemm(q_lat, q_rot, rows, table_row, pos, scale, L: int, n:
 
 
 def _latent_attention_gpu(q_lat, q_rot, rows, block_tables, seq_of, pos, scale, gate, q_lens, ctx_lens, out_dtype,
-                          window: int = 0):
+                          window: int = 0, sink=None):
     T, H, r = q_lat.shape
     f32 = out_dtype == torch.float32
     # sizes the flash kernel cannot hold in LDS / registers: every portion takes the library-product path
@@ -253,13 +258,13 @@ def _latent_attention_gpu(q_lat, q_rot, rows, block_tables, seq_of, pos, scale, 
     big = [b for b, n in enumerate(q_lens) if n >= min_q]
     if not big:
         return _ops().sm_latent_attention(q_lat.contiguous(), q_rot, rows, block_tables, seq_of, pos, scale, gate,
-                                          max(ctx_lens), f32, window)
+                                          max(ctx_lens), f32, window, sink)
     out = torch.empty(T, H, r, dtype=out_dtype, device=q_lat.device)
     small, small_ctx, t0 = [], 1, 0
     for b, (n, L) in enumerate(zip(q_lens, ctx_lens)):
         if n >= min_q:
             o = _latent_attention_gemm(q_lat[t0:t0 + n], q_rot[t0:t0 + n], rows, block_tables[b], pos[t0:t0 + n], scale,
-                                       L, n, window)
+                                       L, n, window, sink)
             if gate is not None:
                 o = o * torch.sigmoid(gate[t0:t0 + n].float())[..., None]
             out[t0:t0 + n] = o.to(out_dtype)
@@ -271,7 +276,7 @@ def _latent_attention_gpu(q_lat, q_rot, rows, block_tables, seq_of, pos, scale, 
         idx = torch.cat(small)
         o = _ops().sm_latent_attention(q_lat[idx].contiguous(), q_rot[idx], rows, block_tables,
                                        seq_of[idx].contiguous(), pos[idx].contiguous(), scale,
-                                       gate[idx] if gate is not None else None, small_ctx, f32, window)
+                                       gate[idx] if gate is not None else None, small_ctx, f32, window, sink)
         out[idx] = o
     return out
 
@@ -431,14 +436,15 @@ def _mlstm_scan_gpu(q, k, v, i_pre, f_pre, i_bias, f_bias, cap, state, cu, state
 
 
 def head_rms_gate(h: torch.Tensor, norm_w: torch.Tensor, gate_pre: torch.Tensor, eps: float,
-                  out_dtype: torch.dtype) -> torch.Tensor:
+                  out_dtype: torch.dtype, silu: bool = False) -> torch.Tensor:
     """h f32 [T, H, dv]: every head divided by its root mean square, then
-    ``* norm_w`` (all heads' size) ``* sigmoid(gate_pre)`` -> [T, H * dv]."""
+    ``* norm_w`` (all heads' size) ``* sigmoid(gate_pre)`` (or ``silu(gate_pre)``) -> [T, H * dv]."""
     T, H, dv = h.shape
     if native(h):
-        return _ops().sm_head_rms_gate(h.contiguous(), norm_w, gate_pre, eps, out_dtype == torch.float32)
+        return _ops().sm_head_rms_gate(h.contiguous(), norm_w, gate_pre, eps, out_dtype == torch.float32, silu)
     y = h * torch.rsqrt((h * h).mean(-1, keepdim=True) + eps)
-    y = y.reshape(T, H * dv) * norm_w.float() * torch.sigmoid(gate_pre.float())
+    g = F.silu(gate_pre.float()) if silu else torch.sigmoid(gate_pre.float())
+    y = y.reshape(T, H * dv) * norm_w.float() * g
     return y.to(out_dtype)
 
 

@@ -26,7 +26,7 @@ import torch.nn.functional as F
 from .seqmix import native
 
 __all__ = ["PairMean", "ExpertSum", "dyn_tanh", "add_normed_", "decay_scan", "delta_scan", "rms_sigmoid_gate",
-           "rglru_gates", "rglru_scan", "route_groups", "route", "SCAN_MAX_DIM"]
+           "rglru_gates", "rglru_scan", "RouteRule", "route_groups", "route", "SCAN_MAX_DIM"]
 
 SCAN_MAX_DIM = 512             # largest key size per head the scan kernels hold (4 lanes x 128 state rows)
 
@@ -252,36 +252,63 @@ def rglru_scan(a: torch.Tensor, x: torch.Tensor, y_pre: torch.Tensor, state: tor
 
 
 # ------------------------------------------------------------------ routing
-def route_groups(z: torch.Tensor, correction: Optional[torch.Tensor], top: int, groups: int,
-                 keep: int) -> Tuple[torch.Tensor, torch.Tensor]:
+@dataclass
+class RouteRule:
+    """How router logits become scores and weights.  ``score``: "softmax" over all router outputs, or "sigmoid";
+    ``group``: a group's score is its "max" corrected score, or the sum of its two largest ("top2"); ``renorm``: the
+    winners' scores are divided by their sum (+ 1e-20) and multiplied by ``scale``."""
+    score: str = "softmax"
+    group: str = "max"
+    renorm: bool = False
+    scale: float = 1.0
+
+    def __post_init__(self):
+        if self.score not in ("softmax", "sigmoid") or self.group not in ("max", "top2"):
+            raise ValueError(f"unknown routing rule {self}")
+        if not self.renorm and self.scale != 1.0:
+            raise ValueError("a routing scale belongs to renormalised weights")
+
+    def args(self):
+        return self.score == "sigmoid", self.group == "top2", self.renorm, float(self.scale)
+
+
+SOFTMAX_RULE = RouteRule()
+
+
+def route_groups(z: torch.Tensor, correction: Optional[torch.Tensor], top: int, groups: int, keep: int,
+                 rule: RouteRule = SOFTMAX_RULE) -> Tuple[torch.Tensor, torch.Tensor]:
     """Router logits ``z`` f32 [T, E] -> the chosen experts (int32 [T, top]) and
-    their weights (f32 [T, top]).  Scores s = softmax(z) over all E; the choice
-    goes by c = s + ``correction`` (f32 [E] or None).  The E experts form
-    ``groups`` equal groups of neighbours; the ``keep`` groups with the largest
-    best c stay, the others' experts cannot be chosen.  The ``top`` largest c
-    win (lowest index first among equals, groups alike); the weights are their
-    s, not renormalised."""
+    their weights (f32 [T, top]).  Scores s = softmax(z) over all E (or sigmoids,
+    ``rule``); the choice goes by c = s + ``correction`` (f32 [E] or None).  The E
+    experts form ``groups`` equal groups of neighbours; the ``keep`` groups with
+    the largest best c (or sum of the two best) stay, the others' experts cannot
+    be chosen.  The ``top`` largest c win (lowest index first among equals, groups
+    alike); the weights are their s, as they are or renormalised."""
     T, E = z.shape
     if native(z) and E <= 512:
-        return _ops().sx_route_groups(z.contiguous(), correction, top, groups, keep)
-    s = torch.softmax(z.float(), -1)
+        return _ops().sx_route_groups(z.contiguous(), correction, top, groups, keep, *rule.args())
+    s = torch.sigmoid(z.float()) if rule.score == "sigmoid" else torch.softmax(z.float(), -1)
     c = s + correction.float() if correction is not None else s
     if keep < groups:
-        best = c.view(T, groups, E // groups).max(-1).values
+        n = min(2 if rule.group == "top2" else 1, E // groups)
+        best = c.view(T, groups, E // groups).topk(n, -1).values.sum(-1)
         kept = torch.sort(best, dim=-1, descending=True, stable=True).indices[:, :keep]
         ok = torch.zeros(T, groups, dtype=torch.bool, device=z.device).scatter_(1, kept, True)
         c = c.masked_fill(~ok.repeat_interleave(E // groups, 1), float("-inf"))
     idx = torch.sort(c, dim=-1, descending=True, stable=True).indices[:, :top]
-    return idx.to(torch.int32).contiguous(), s.gather(1, idx).contiguous()
+    w = s.gather(1, idx)
+    if rule.renorm:
+        w = w * (rule.scale / (w.sum(-1, keepdim=True) + 1e-20))
+    return idx.to(torch.int32).contiguous(), w.contiguous()
 
 
 ROUTER_MAX_T = 64              # GPU: up to this many tokens the logits and the routing are one launch
 
 
 def route(h: torch.Tensor, router: torch.Tensor, correction: Optional[torch.Tensor], top: int, groups: int,
-          keep: int) -> Tuple[torch.Tensor, torch.Tensor]:
+          keep: int, rule: RouteRule = SOFTMAX_RULE) -> Tuple[torch.Tensor, torch.Tensor]:
     """``route_groups`` of the logits ``h router^T`` (f32 products; ``h`` [T, W] in the activation dtype, ``router``
     f32 [E, W])"""
     if native(h) and h.shape[0] <= ROUTER_MAX_T and router.shape[0] <= 512:
-        return _ops().sx_router(h.contiguous(), router, correction, top, groups, keep)
-    return route_groups(F.linear(h.float(), router), correction, top, groups, keep)
+        return _ops().sx_router(h.contiguous(), router, correction, top, groups, keep, *rule.args())
+    return route_groups(F.linear(h.float(), router), correction, top, groups, keep, rule)
