@@ -194,7 +194,19 @@ def main():
     ap.add_argument("--sandwich-sizes", default="small,base")
     ap.add_argument("--sandwich-prompts", default="1024,4096")
     ap.add_argument("--no-sandwich-ref", action="store_true", help="--sandwich: skip the comparison model")
+    ap.add_argument("--looped", action="store_true",
+                    help="side benchmark (not the headline metric): prefill / decode throughput of the pre-norm decoder "
+                         "whose middle layers run twice (delta rule with per-channel decays, latent attention with a sink, "
+                         "causal attention beside time mixing, experts behind a sigmoid router) beside the decoder normed "
+                         "before and after every sublayer at equal sizes, one GPU")
+    ap.add_argument("--looped-sizes", default="small,base")
+    ap.add_argument("--looped-prompts", default="1024,4096")
+    ap.add_argument("--no-looped-ref", action="store_true", help="--looped: skip the comparison model")
     args = ap.parse_args()
+    if args.looped:
+        from ipex_llm_amd.utils.bench_looped import main as looped_main
+        looped_main(args)
+        return
     if args.sandwich:
         from ipex_llm_amd.utils.bench_sandwich import main as sandwich_main
         sandwich_main(args)
