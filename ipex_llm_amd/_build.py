@@ -97,7 +97,7 @@ def _cmd(src: str, obj: str):
 TARGETS = {
     # hybrid decoders: sequence-mixing kernels + their bindings + the serving scheduler
     # (+ the streaming skinny-GEMM kernel their decode-size projections share with the dense decoders)
-    "seqmix": ["hip/seqmix.hip", "hip/blockmix_elem.hip", "hip/blockmix_attn.hip", "hip/blockmix_moe.hip",
+    "seqmix": ["hip/seqmix.hip", "hip/latent_decode.hip", "hip/blockmix_elem.hip", "hip/blockmix_attn.hip", "hip/blockmix_moe.hip",
                "hip/ssm.hip", "hip/maskattn.hip", "hip/gatedmix.hip", "hip/statemix.hip",
                "hip/statemix_scan.hip", "hip/statemix_chunk.hip", "hip/chanmix.hip", "hip/chanmix_scan.hip",
                "hip/chanmix_chunk.hip", "hip/dense_gemv.hip", "torch/ops_seqmix.cpp",

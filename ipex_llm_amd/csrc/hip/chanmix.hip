@@ -215,66 +215,103 @@ __global__ void __launch_bounds__(256) last_rows_k(const E* __restrict__ h, floa
 }
 
 // ------------------------------------------------------------------ low-rank decay
-__device__ __forceinline__ float softplusf(float z) { return z > 20.f ? z : log1pf(expf(z)); }
+// softplus(z) = max(z, 0) + log1p(t), t = exp(-|z|); log1p(t) = 2 atanh(s), s = t / (2 + t) <= 1/3, by its power series
+__device__ __forceinline__ float softplusf(float z) {
+  const float t = __expf(-fabsf(z)), s = t / (2.0f + t), q = s * s;
+  float a = 1.0f / 15.0f;
+  a = fmaf(a, q, 1.0f / 13.0f);
+  a = fmaf(a, q, 1.0f / 11.0f);
+  a = fmaf(a, q, 1.0f / 9.0f);
+  a = fmaf(a, q, 1.0f / 7.0f);
+  a = fmaf(a, q, 1.0f / 5.0f);
+  a = fmaf(a, q, 1.0f / 3.0f);
+  a = fmaf(a, q, 1.0f);
+  return fmaxf(z, 0.f) + 2.0f * s * a;
+}
 
 // the parts of an input value: tanh leaves an f32 number (three 16-bit parts), a plain 16-bit input is one part
 template <typename E, bool SQ> struct InParts { static constexpr int N = 1; };
 template <> struct InParts<__bf16, true> { static constexpr int N = 3; };
 
-// a workgroup: TM tokens x 64 outputs, wave w the outputs 16 w .. 16 w + 15; inside a step of 32 lane group g holds
-// k = 8 g .. 8 g + 7 (inputs and weights alike, so the f32 products may take them one after another)
-template <typename E, int TM, bool SQ>
+// a workgroup: TM tokens x 64 NT outputs, wave w the NT tiles of 16 from 16 NT w on; inside a step of 32 lane group g
+// holds k = 8 g .. 8 g + 7 (inputs and weights alike, so the f32 products may take them one after another)
+template <typename E, int TM, int NT, bool SQ>
 __global__ void __launch_bounds__(256) lowrank_decay_k(const E* __restrict__ in, int64_t ld, const E* __restrict__ w,
                                                       const float* __restrict__ rate, const float* __restrict__ bias,
                                                       int kind, float* __restrict__ out, int T, int N, int R) {
-  constexpr int NP = InParts<E, SQ>::N, KC = 32, LP = KC + (sizeof(E) == 2 ? 8 : 4), MS = TM / 16;
+  constexpr int NP = InParts<E, SQ>::N, KC = 64, LP = KC + (sizeof(E) == 2 ? 8 : 4), MS = TM / 16;
   __shared__ __attribute__((aligned(16))) E us[NP][TM * LP];
   const int t0 = blockIdx.x * TM;
   const int tid = threadIdx.x, wv = tid >> 6, lane = tid & 63, r16 = lane & 15, g = lane >> 4;
-  const int n = blockIdx.y * 64 + 16 * wv + r16;
-  const bool ok = n < N;
-  const E* wr = w + (int64_t)(ok ? n : 0) * R;
+  const int n0 = (blockIdx.y * 4 + wv) * 16 * NT + r16;
   const bool vec = R % 8 == 0;
-  f32x4 acc[MS];
+  f32x4 acc[NT][MS];
 #pragma unroll
-  for (int m = 0; m < MS; m++) acc[m] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int c = 0; c < NT; c++)
+#pragma unroll
+    for (int m = 0; m < MS; m++) acc[c][m] = f32x4{0.f, 0.f, 0.f, 0.f};
   for (int k0 = 0; k0 < R; k0 += KC) {
-    sx::Frag<E> b;
-    b.load(wr, k0 + 8 * g, ok ? R : 0, vec);
+    sx::Frag<E> b[NT][KC / 32];
+#pragma unroll
+    for (int c = 0; c < NT; c++) {
+      const int n = n0 + 16 * c;
+#pragma unroll
+      for (int ks = 0; ks < KC / 32; ks++)
+        b[c][ks].load(w + (int64_t)(n < N ? n : 0) * R, k0 + 32 * ks + 8 * g, n < N ? R : 0, vec);
+    }
     __syncthreads();
-    for (int i = tid; i < TM * KC; i += 256) {
-      const int r = i / KC, c = i - r * KC;
-      float v = (t0 + r < T && k0 + c < R) ? ldf(in + (int64_t)(t0 + r) * ld + k0 + c) : 0.f;
-      if (SQ) v = tanhf(v);
+    constexpr int PER = TM * KC / 256;                              // values per thread, all requested together
+    float x[PER];
+#pragma unroll
+    for (int j = 0; j < PER; j++) {
+      const int i = tid + 256 * j, r = i / KC, c = i - r * KC;
+      x[j] = (t0 + r < T && k0 + c < R) ? ldf(in + (int64_t)(t0 + r) * ld + k0 + c) : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < PER; j++) {
+      const int i = tid + 256 * j, r = i / KC, c = i - r * KC;
+      const float v = SQ ? tanhf(x[j]) : x[j];
       if constexpr (NP == 3) sx::stage(us, r * LP + c, v);
       else us[0][r * LP + c] = (E)v;
     }
     __syncthreads();
 #pragma unroll
-    for (int m = 0; m < MS; m++) {
+    for (int ks = 0; ks < KC / 32; ks++) {
+      if (k0 + 32 * ks >= R) break;
 #pragma unroll
-      for (int p = NP - 1; p >= 0; p--) {                           // smallest part first
-        const E* up = us[p] + (m * 16 + r16) * LP + 8 * g;
-        if constexpr (sizeof(E) == 2) {
-          acc[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)up, b.v8(), acc[m], 0, 0, 0);
-        } else {
+      for (int m = 0; m < MS; m++) {
 #pragma unroll
-          for (int j = 0; j < 8; j++) acc[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(up[j], b.v[j], acc[m], 0, 0, 0);
+        for (int p = NP - 1; p >= 0; p--) {                         // smallest part first
+          const E* up = us[p] + (m * 16 + r16) * LP + 32 * ks + 8 * g;
+#pragma unroll
+          for (int c = 0; c < NT; c++) {
+            if constexpr (sizeof(E) == 2) {
+              acc[c][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)up, b[c][ks].v8(), acc[c][m], 0, 0, 0);
+            } else {
+#pragma unroll
+              for (int j = 0; j < 8; j++)
+                acc[c][m] = __builtin_amdgcn_mfma_f32_16x16x4f32(up[j], b[c][ks].v[j], acc[c][m], 0, 0, 0);
+            }
+          }
         }
       }
     }
   }
-  if (!ok) return;
-  const float bs = bias[n], rt = kind == 0 ? rate[n] : 0.f;
 #pragma unroll
-  for (int m = 0; m < MS; m++)
+  for (int c = 0; c < NT; c++) {
+    const int n = n0 + 16 * c;
+    if (n >= N) continue;
+    const float bs = bias[n], rt = kind == 0 ? rate[n] : 0.f;
 #pragma unroll
-    for (int i = 0; i < 4; i++) {
-      const int t = t0 + m * 16 + 4 * g + i;
-      if (t >= T) continue;
-      const float z = acc[m][i] + bs;
-      out[(int64_t)t * N + n] = kind == 0 ? expf(-rt * softplusf(z)) : expf(-expf(z));
-    }
+    for (int m = 0; m < MS; m++)
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        const int t = t0 + m * 16 + 4 * g + i;
+        if (t >= T) continue;
+        const float z = acc[c][m][i] + bs;
+        out[(int64_t)t * N + n] = kind == 0 ? __expf(-rt * softplusf(z)) : __expf(-__expf(z));
+      }
+  }
 }
 
 // ------------------------------------------------------------------ grouped skinny product
@@ -400,11 +437,11 @@ void token_mixes(bool bf16, const void* h, const float* mu, int NM, float* state
 void lowrank_decay(bool bf16, const void* in, int64_t ld, const void* w, const float* rate, const float* bias, int kind,
                    bool squash, float* out, int T, int N, int R, hipStream_t st) {
   if (T <= 0 || N <= 0) return;
-#define CALL(E, TM, SQ)                                                                                             \
-  lowrank_decay_k<E, TM, SQ><<<dim3((T + TM - 1) / TM, (N + 63) / 64), 256, 0, st>>>((const E*)in, ld, (const E*)w, rate, \
-                                                                                     bias, kind, out, T, N, R)
+#define CALL(E, TM, NT, SQ)                                                                                        \
+  lowrank_decay_k<E, TM, NT, SQ><<<dim3((T + TM - 1) / TM, (N + 64 * NT - 1) / (64 * NT)), 256, 0, st>>>(            \
+      (const E*)in, ld, (const E*)w, rate, bias, kind, out, T, N, R)
 #define CALL_T(E, SQ) \
-  if (T <= 64) CALL(E, 16, SQ); else CALL(E, 64, SQ)
+  if (T <= 64) CALL(E, 16, 1, SQ); else CALL(E, 64, 2, SQ)
   if (bf16) { if (squash) { CALL_T(__bf16, true); } else { CALL_T(__bf16, false); } }
   else { if (squash) { CALL_T(float, true); } else { CALL_T(float, false); } }
 #undef CALL_T

@@ -145,8 +145,9 @@ __global__ void __launch_bounds__(1024) qkv_store_k(const EI* __restrict__ q, in
     for (int e = threadIdx.x; e < G * dv; e += blockDim.x) stf(row + (int64_t)G * d + e, ldf(v + t * v_ld + e));
 }
 
-// the same step for per-head norms (or none) and neighbouring pairs: eight neighbouring values per lane, LPH lanes per
-// head (a power of two), 64 / LPH heads per wave, every value read once (d and dv multiples of 8, d <= 8 LPH)
+// the same step for per-head norms (or none): eight neighbouring values per lane, LPH lanes per head (a power of two),
+// 64 / LPH heads per wave, every value read once (d and dv multiples of 8, d <= 8 LPH).  HALF: half-split pairs (dims a
+// multiple of 16: a value's partner sits in the same place of another lane), otherwise neighbouring pairs
 template <typename E> struct Eight {
   typedef E V8 __attribute__((ext_vector_type(8)));
   static __device__ __forceinline__ void ld(const E* p, float* v) {
@@ -162,7 +163,7 @@ template <typename E> struct Eight {
   }
 };
 
-template <typename EI, typename E, int LPH>
+template <typename EI, typename E, int LPH, bool HALF>
 __global__ void __launch_bounds__(512) qkv_store_pairs_k(const EI* __restrict__ q, int64_t q_ld, const EI* __restrict__ k,
                                                         int64_t k_ld, const EI* __restrict__ v, int64_t v_ld,
                                                         const E* __restrict__ qn, const E* __restrict__ kn, float eps,
@@ -174,9 +175,18 @@ __global__ void __launch_bounds__(512) qkv_store_pairs_k(const EI* __restrict__ 
   const int ln = threadIdx.x & (LPH - 1), i0 = 8 * ln;
   const int NK = H + (k ? G : 0), per = blockDim.x / LPH;           // heads per pass
   E* row = k ? rows + slots[t] * ((int64_t)G * (d + dv)) : nullptr;
-  float cs[8];                                                      // this lane's four pairs: (cos, sin)
+  float cs[HALF ? 16 : 8];                                          // this lane's pairs: (cos, sin)
   const bool turn = table && i0 < dims;
-  if (turn) {
+  const bool first = i0 < dims / 2;                                 // half-split: the pairs' first values
+  const int mate = (threadIdx.x & 63) + (turn ? (first ? dims / 16 : -dims / 16) : 0);
+  if (HALF && turn) {
+    const float* p = table + pos[t] * dims + 2 * (first ? i0 : i0 - dims / 2);
+#pragma unroll
+    for (int i = 0; i < 16; i += 4) {
+      const float4 r = *(const float4*)(p + i);
+      cs[i] = r.x, cs[i + 1] = r.y, cs[i + 2] = r.z, cs[i + 3] = r.w;
+    }
+  } else if (turn) {
     const float* p = table + pos[t] * dims + i0;
 #pragma unroll
     for (int i = 0; i < 8; i += 2) {
@@ -191,6 +201,8 @@ __global__ void __launch_bounds__(512) qkv_store_pairs_k(const EI* __restrict__ 
     const int hh = h0 + threadIdx.x / LPH;
     const bool isq = hh < H, ok = in && hh < NK;
     float a[8];
+#pragma unroll
+    for (int i = 0; i < 8; i++) a[i] = 0.f;
     float ss = 0.f;
     if (ok) {
       Eight<EI>::ld(isq ? q + t * q_ld + (int64_t)hh * d + i0 : k + t * k_ld + (int64_t)(hh - H) * d + i0, a);
@@ -201,16 +213,21 @@ __global__ void __launch_bounds__(512) qkv_store_pairs_k(const EI* __restrict__ 
 #pragma unroll
       for (int o = LPH / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
     }
-    if (!ok) continue;
     const E* nw = isq ? qn : kn;
-    if (nw) {
+    if (ok && nw) {
       const float rs = 1.0f / sqrtf(ss / (float)d + eps);
       float w[8];
       Eight<E>::ld(nw + i0, w);
 #pragma unroll
       for (int i = 0; i < 8; i++) a[i] = a[i] * rs * w[i];
     }
-    if (turn) {
+    if (HALF) {                                                     // (every lane takes part in the exchange)
+#pragma unroll
+      for (int i = 0; i < 8; i++) {
+        const float other = __shfl(a[i], mate, 64);
+        if (turn) a[i] = first ? a[i] * cs[2 * i] - other * cs[2 * i + 1] : a[i] * cs[2 * i] + other * cs[2 * i + 1];
+      }
+    } else if (turn) {
 #pragma unroll
       for (int i = 0; i < 8; i += 2) {
         const float n0 = a[i] * cs[i] - a[i + 1] * cs[i + 1];
@@ -218,6 +235,7 @@ __global__ void __launch_bounds__(512) qkv_store_pairs_k(const EI* __restrict__ 
         a[i] = n0;
       }
     }
+    if (!ok) continue;
     if (isq) {
       if (temp) {
         const float f = temp[hh];
@@ -557,7 +575,8 @@ __global__ void __launch_bounds__(64) talk_mix_k(const float* __restrict__ w, co
 // sliding window: query tok stands at position q0 + tok; the first nkeep columns are kept first tokens (always
 // visible), column nkeep + jj is the key at position k0 + jj, visible when it is not ahead of the query and inside
 // the window (or before position ``keep``)
-template <typename E>
+// KEEP > 0: 4-value accesses, the row stays in registers between the passes (L a multiple of 4, at most 1024 KEEP)
+template <typename E, int KEEP>
 __global__ void __launch_bounds__(256) chunk_softmax_k(float* __restrict__ sc, int Lq, int L, int G, int rep, float scale,
                                                       const float* __restrict__ sink, E* __restrict__ hi, float softcap,
                                                       int window, int keep, int nkeep, int64_t q0, int64_t k0) {
@@ -573,12 +592,32 @@ __global__ void __launch_bounds__(256) chunk_softmax_k(float* __restrict__ sc, i
   float* s = sc + row * L;
   const float sk = sink ? sink[h] : -INFINITY;
   float mx = sk;
-  for (int j = threadIdx.x; j < nk; j += blockDim.x) {
-    float v = s[j] * scale;
-    if (softcap > 0.f) v = softcap * tanhf(v / softcap);
-    if (!vis(j)) v = -INFINITY;
-    s[j] = v;
-    mx = fmaxf(mx, v);
+  constexpr int NK = KEEP > 0 ? KEEP : 1;
+  float v[NK][4];
+  auto cap = [&](float x) { return softcap > 0.f ? softcap * tanhf(x / softcap) : x; };
+  if (KEEP > 0) {
+#pragma unroll
+    for (int k = 0; k < KEEP; k++) {
+      const int j = 4 * (threadIdx.x + 256 * k);
+#pragma unroll
+      for (int i = 0; i < 4; i++) v[k][i] = -INFINITY;
+      if (j < nk) {
+        const float4 a = *(const float4*)(s + j);
+        const float t[4] = {a.x, a.y, a.z, a.w};
+#pragma unroll
+        for (int i = 0; i < 4; i++)
+          if (j + i < nk && vis(j + i)) {
+            v[k][i] = cap(t[i] * scale);
+            mx = fmaxf(mx, v[k][i]);
+          }
+      }
+    }
+  } else {
+    for (int j = threadIdx.x; j < nk; j += blockDim.x) {
+      const float x = vis(j) ? cap(s[j] * scale) : -INFINITY;
+      s[j] = x;
+      mx = fmaxf(mx, x);
+    }
   }
   mx = wave_max(mx);
   __syncthreads();
@@ -586,12 +625,45 @@ __global__ void __launch_bounds__(256) chunk_softmax_k(float* __restrict__ sc, i
   __syncthreads();
   for (int i = 0; i < (int)(blockDim.x >> 6); i++) mx = fmaxf(mx, red[i]);
   float sum = 0.f;
-  for (int j = threadIdx.x; j < nk; j += blockDim.x) {
-    const float e = expf(s[j] - mx);                               // a masked column: exp(-inf) = 0
-    s[j] = e;
-    sum += e;
+  if (KEEP > 0) {
+#pragma unroll
+    for (int k = 0; k < KEEP; k++)
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        v[k][i] = expf(v[k][i] - mx);                              // a masked column: exp(-inf) = 0
+        sum += v[k][i];
+      }
+  } else {
+    for (int j = threadIdx.x; j < nk; j += blockDim.x) {
+      const float e = expf(s[j] - mx);
+      s[j] = e;
+      sum += e;
+    }
   }
   const float inv = 1.0f / (block_sum(sum, red) + (sink ? expf(sk - mx) : 0.f));
+  if (KEEP > 0) {
+#pragma unroll
+    for (int k = 0; k < KEEP; k++) {
+      const int j = 4 * (threadIdx.x + 256 * k);
+      if (j >= L) continue;
+#pragma unroll
+      for (int i = 0; i < 4; i++) v[k][i] *= inv;
+      if (hi) {                                                     // [R, 2 L]: hi halves, then lo halves
+        typedef E E4 __attribute__((ext_vector_type(4)));
+        E4 h4, l4;
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+          h4[i] = (E)v[k][i];
+          l4[i] = (E)(v[k][i] - (float)h4[i]);
+        }
+        *(E4*)(hi + row * 2 * L + j) = h4;
+        *(E4*)(hi + row * 2 * L + L + j) = l4;
+      } else {
+        *(float4*)(s + j) = make_float4(v[k][0], v[k][1], v[k][2], v[k][3]);
+      }
+    }
+    return;
+  }
   for (int j = threadIdx.x; j < L; j += blockDim.x) {
     const float w = j < nk ? s[j] * inv : 0.f;
     if (hi) {                                                      // [R, 2 L]: hi halves, then lo halves
@@ -646,7 +718,8 @@ void qkv_norm_rope_store(bool in_bf16, bool bf16, const void* q, int64_t q_ld, c
   if (T <= 0) return;
   const size_t ei = in_bf16 ? 2 : 4, eo = bf16 ? 2 : 4;
   auto wide = [](const void* p, int64_t ld, size_t eb) { return (uintptr_t)p % (8 * eb) == 0 && ld % 8 == 0; };
-  if (!whole && (!table || layout != kHalf) && d % 8 == 0 && d <= 512 && wide(q, q_ld, ei) && wide(qn, 0, eo) &&
+  const bool half = table && layout == kHalf;
+  if (!whole && (!half || dims % 16 == 0) && d % 8 == 0 && d <= 512 && wide(q, q_ld, ei) && wide(qn, 0, eo) &&
       wide(kn, 0, eo) && (!k || (dv % 8 == 0 && wide(k, k_ld, ei) && wide(v, v_ld, ei) && wide(rows, 0, eo)))) {
     int lph = 1;
     while (8 * lph < d) lph *= 2;
@@ -654,7 +727,9 @@ void qkv_norm_rope_store(bool in_bf16, bool bf16, const void* q, int64_t q_ld, c
     nt = (nt + 63) / 64 * 64;
     nt = T > 64 ? (nt > 256 ? 256 : nt) : (nt > 512 ? 512 : nt);
 #define MA_PAIRS(EI, E, L)                                                                                              \
-  qkv_store_pairs_k<EI, E, L><<<T, nt, 0, st>>>((const EI*)q, q_ld, (const EI*)k, k_ld, (const EI*)v, v_ld,             \
+  if (half) MA_PAIRS_H(EI, E, L, true); else MA_PAIRS_H(EI, E, L, false)
+#define MA_PAIRS_H(EI, E, L, HF)                                                                                        \
+  qkv_store_pairs_k<EI, E, L, HF><<<T, nt, 0, st>>>((const EI*)q, q_ld, (const EI*)k, k_ld, (const EI*)v, v_ld,             \
                                                 (const E*)qn, (const E*)kn, eps, table, dims, pos, slots, (E*)rows, qo, \
                                                 temp, H, G, d, dv)
 #define MA_L(EI, E)                      \
@@ -672,6 +747,7 @@ void qkv_norm_rope_store(bool in_bf16, bool bf16, const void* q, int64_t q_ld, c
     else { MA_L(float, float) }
 #undef MA_L
 #undef MA_PAIRS
+#undef MA_PAIRS_H
     return;
   }
   const size_t lds = (size_t)(H + G + 2) * sizeof(float);
@@ -765,12 +841,16 @@ void masked_attention(bool bf16, const float* q, const void* rows, int bs, const
 void chunk_softmax(bool bf16, float* sc, int64_t R, int Lq, int L, int G, int rep, float scale, const float* sink,
                    void* hl, float softcap, int window, int keep, int nkeep, int64_t q0, int64_t k0, hipStream_t st) {
   if (R <= 0 || L <= 0) return;
-  if (bf16)
-    chunk_softmax_k<__bf16><<<(unsigned)R, 256, 0, st>>>(sc, Lq, L, G, rep, scale, sink, (__bf16*)hl, softcap, window,
-                                                         keep, nkeep, q0, k0);
-  else
-    chunk_softmax_k<float><<<(unsigned)R, 256, 0, st>>>(sc, Lq, L, G, rep, scale, sink, (float*)nullptr, softcap, window,
-                                                        keep, nkeep, q0, k0);
+#define MA_SOFT(E, K) \
+  chunk_softmax_k<E, K><<<(unsigned)R, 256, 0, st>>>(sc, Lq, L, G, rep, scale, sink, (E*)hl, softcap, window, keep, nkeep, q0, k0)
+  if (L % 4 == 0 && L <= 2048) {
+    if (bf16) MA_SOFT(__bf16, 2); else MA_SOFT(float, 2);
+  } else if (L % 4 == 0 && L <= 4096) {
+    if (bf16) MA_SOFT(__bf16, 4); else MA_SOFT(float, 4);
+  } else {
+    if (bf16) MA_SOFT(__bf16, 0); else MA_SOFT(float, 0);
+  }
+#undef MA_SOFT
 }
 
 void talk_mix(bool bf16, const float* w, const float* talk, int64_t pieces, int Lq, int L, int G, int rep, void* hl,

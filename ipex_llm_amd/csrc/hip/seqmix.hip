@@ -120,7 +120,7 @@ __global__ void __launch_bounds__(256) layer_norm_k(const float* __restrict__ x,
 
 // ------------------------------------------------------------------ rotary
 template <typename E>
-__global__ void __launch_bounds__(256) rope_rows_k(E* __restrict__ q, int H, int Dh, int offset,
+__global__ void __launch_bounds__(256) rope_rows_k(E* __restrict__ q, int64_t st, int64_t sh, int H, int offset,
                                                   const float* __restrict__ table, int max_pos, int dims,
                                                   const int64_t* __restrict__ pos) {
   const int64_t t = blockIdx.x;
@@ -130,7 +130,7 @@ __global__ void __launch_bounds__(256) rope_rows_k(E* __restrict__ q, int H, int
   const float* cs = table + p * dims;             // [half][2]
   for (int i = threadIdx.x; i < H * half; i += blockDim.x) {
     const int h = i / half, k = i - h * half;
-    E* a = q + (t * H + h) * Dh + offset + 2 * k;
+    E* a = q + t * st + h * sh + offset + 2 * k;
     const float u = ldf(a), v = ldf(a + 1), c = cs[2 * k], s = cs[2 * k + 1];
     stf(a, u * c - v * s);
     stf(a + 1, v * c + u * s);
@@ -633,40 +633,96 @@ __global__ void __launch_bounds__(128) latent_attn_combine_k(const float* __rest
 // belongs to query token i / H at position pos[i / H]; keys j <= pos get
 // softmax(scale * s) in f32, the others 0.  E = float: written in place.
 // E = bf16: the f32 weight leaves as a pair of bf16 values hi + lo (hi the
-// rounded weight, lo the rounded remainder), so the following bf16 products
-// carry the weights to ~2^-17 instead of 2^-9.
-template <typename E>
-__global__ void __launch_bounds__(256) causal_softmax_k(float* __restrict__ sc, int64_t ld, const int64_t* __restrict__ pos,
-                                                       int H, float scale, int L, E* __restrict__ hi, E* __restrict__ lo,
-                                                       int64_t key0, int window, const float* __restrict__ sink) {
+// rounded weight, lo the rounded remainder; hl [R, 2 L]: hi halves, then lo
+// halves), so the following bf16 product carries the weights to ~2^-17 instead
+// of 2^-9.  V = 4, KEEP > 0: 4-value accesses, the row stays in registers between
+// the passes (L a multiple of 4, at most 1024 KEEP); otherwise it is read again.
+template <typename E, int V, int KEEP>
+__global__ void __launch_bounds__(256) causal_softmax_k(float* __restrict__ sc, const int64_t* __restrict__ pos, int H,
+                                                       float scale, int L, E* __restrict__ hl, int64_t key0, int window,
+                                                       const float* __restrict__ sink) {
   __shared__ float red[16];
   const int64_t row = blockIdx.x;
   const int64_t p = pos[row / H];
   // column j is key key0 + j; visible: key <= p, and key > p - window with a window
   const int nk = (int)max((int64_t)0, min((int64_t)L, p - key0 + 1));
   const int j0 = window > 0 ? (int)max((int64_t)0, min((int64_t)nk, p - window + 1 - key0)) : 0;
-  float* s = sc + row * ld;
+  float* s = sc + row * L;
   const float sk = sink ? sink[row % H] : -INFINITY;
   float mx = sk;
-  for (int j = j0 + threadIdx.x; j < nk; j += blockDim.x) mx = fmaxf(mx, s[j] * scale);
+  constexpr int NK = KEEP > 0 ? KEEP : 1;
+  float v[NK][4];
+  if (KEEP > 0) {
+#pragma unroll
+    for (int k = 0; k < KEEP; k++) {
+      const int j = 4 * (threadIdx.x + 256 * k);
+#pragma unroll
+      for (int i = 0; i < 4; i++) v[k][i] = -INFINITY;
+      if (j < nk && j + 3 >= j0) {
+        const float4 a = *(const float4*)(s + j);
+        const float t[4] = {a.x, a.y, a.z, a.w};
+#pragma unroll
+        for (int i = 0; i < 4; i++)
+          if (j + i >= j0 && j + i < nk) {
+            v[k][i] = t[i] * scale;
+            mx = fmaxf(mx, v[k][i]);
+          }
+      }
+    }
+  } else {
+    for (int j = j0 + threadIdx.x; j < nk; j += blockDim.x) mx = fmaxf(mx, s[j] * scale);
+  }
   mx = wave_max(mx);
   __syncthreads();
   if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = mx;
   __syncthreads();
   for (int i = 0; i < (int)(blockDim.x >> 6); i++) mx = fmaxf(mx, red[i]);
   float sum = 0.f;
-  for (int j = j0 + threadIdx.x; j < nk; j += blockDim.x) {
-    const float e = expf(s[j] * scale - mx);
-    s[j] = e;
-    sum += e;
+  if (KEEP > 0) {
+#pragma unroll
+    for (int k = 0; k < KEEP; k++)
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        v[k][i] = v[k][i] == -INFINITY ? 0.f : expf(v[k][i] - mx);
+        sum += v[k][i];
+      }
+  } else {
+    for (int j = j0 + threadIdx.x; j < nk; j += blockDim.x) {
+      const float e = expf(s[j] * scale - mx);
+      s[j] = e;
+      sum += e;
+    }
   }
   const float inv = 1.0f / (block_sum(sum, red) + (sink ? expf(sk - mx) : 0.f));
+  if (KEEP > 0) {
+#pragma unroll
+    for (int k = 0; k < KEEP; k++) {
+      const int j = 4 * (threadIdx.x + 256 * k);
+      if (j >= L) continue;
+#pragma unroll
+      for (int i = 0; i < 4; i++) v[k][i] *= inv;
+      if (hl) {
+        typedef E E4 __attribute__((ext_vector_type(4)));
+        E4 hi, lo;
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+          hi[i] = (E)v[k][i];
+          lo[i] = (E)(v[k][i] - (float)hi[i]);
+        }
+        *(E4*)(hl + row * 2 * L + j) = hi;
+        *(E4*)(hl + row * 2 * L + L + j) = lo;
+      } else {
+        *(float4*)(s + j) = make_float4(v[k][0], v[k][1], v[k][2], v[k][3]);
+      }
+    }
+    return;
+  }
   for (int j = threadIdx.x; j < L; j += blockDim.x) {
     const float w = j >= j0 && j < nk ? s[j] * inv : 0.f;
-    if (hi) {
+    if (hl) {
       const E h = (E)w;
-      hi[row * ld + j] = h;
-      lo[row * ld + j] = (E)(w - (float)h);
+      hl[row * 2 * L + j] = h;
+      hl[row * 2 * L + L + j] = (E)(w - (float)h);
     } else {
       s[j] = w;
     }
@@ -921,11 +977,11 @@ void layer_norm(bool bf16, const float* x, const void* w, void* out, int T, int 
   SM_DISPATCH(bf16, hipLaunchKernelGGL(layer_norm_k<E>, dim3(T), dim3(256), 0, st, x, (const E*)w, (E*)out, W, eps));
 }
 
-void rope_rows(bool bf16, void* q, int T, int H, int Dh, int offset, const float* table, int max_pos, int dims,
+void rope_rows(bool bf16, void* q, int64_t st_t, int64_t st_h, int T, int H, int offset, const float* table, int max_pos, int dims,
                const int64_t* pos, hipStream_t st) {
   if (T <= 0) return;
-  SM_DISPATCH(bf16, hipLaunchKernelGGL(rope_rows_k<E>, dim3(T), dim3(256), 0, st, (E*)q, H, Dh, offset, table, max_pos,
-                                       dims, pos));
+  SM_DISPATCH(bf16, hipLaunchKernelGGL(rope_rows_k<E>, dim3(T), dim3(256), 0, st, (E*)q, st_t, st_h, H, offset, table,
+                                       max_pos, dims, pos));
 }
 
 void latent_kv_store(bool bf16, const void* dkv, int64_t ld, const void* norm_w, float eps, int rank, int rot_dim,
@@ -1060,16 +1116,19 @@ void latent_attention(bool bf16, const void* q_lat, const void* q_rot, int64_t q
   }
 }
 
-void causal_softmax(bool bf16, float* sc, int64_t ld, const int64_t* pos, int H, float scale, int64_t R, int L, void* hi,
-                    void* lo, int64_t key0, int window, const float* sink, hipStream_t st) {
+void causal_softmax(bool bf16, float* sc, const int64_t* pos, int H, float scale, int64_t R, int L, void* hl,
+                    int64_t key0, int window, const float* sink, hipStream_t st) {
   if (R <= 0 || L <= 0) return;
-  if (bf16) {
-    hipLaunchKernelGGL(causal_softmax_k<__bf16>, dim3((unsigned)R), dim3(256), 0, st, sc, ld, pos, H, scale, L,
-                       (__bf16*)hi, (__bf16*)lo, key0, window, sink);
+#define SM_SOFT(E, V, K) \
+  causal_softmax_k<E, V, K><<<(unsigned)R, 256, 0, st>>>(sc, pos, H, scale, L, (E*)hl, key0, window, sink)
+  if (L % 4 == 0 && L <= 2048) {
+    if (bf16) SM_SOFT(__bf16, 4, 2); else SM_SOFT(float, 4, 2);
+  } else if (L % 4 == 0 && L <= 4096) {
+    if (bf16) SM_SOFT(__bf16, 4, 4); else SM_SOFT(float, 4, 4);
   } else {
-    hipLaunchKernelGGL(causal_softmax_k<float>, dim3((unsigned)R), dim3(256), 0, st, sc, ld, pos, H, scale, L,
-                       (float*)nullptr, (float*)nullptr, key0, window, sink);
+    if (bf16) SM_SOFT(__bf16, 1, 0); else SM_SOFT(float, 1, 0);
   }
+#undef SM_SOFT
 }
 
 void mlstm_scan(bool bf16, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld,

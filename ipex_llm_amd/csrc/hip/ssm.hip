@@ -126,6 +126,64 @@ __global__ void __launch_bounds__(256) conv_silu_k(const E* __restrict__ u, int6
   }
 }
 
+// the same for long steps: four channels x up to TB neighbouring tokens per thread, the taps and the last inputs in
+// registers (the same sums in the same order)
+constexpr int TB = 8;
+template <typename E, int TAPS, bool ACT>
+__global__ void __launch_bounds__(256) conv_block_k(const E* __restrict__ u, int64_t u_ld, const float* __restrict__ w,
+                                                   const float* __restrict__ bias, const float* __restrict__ state,
+                                                   const int32_t* __restrict__ cu, const int32_t* __restrict__ seq_of,
+                                                   const int32_t* __restrict__ slots, const int64_t* __restrict__ pos,
+                                                   float* __restrict__ out, int T, int C) {
+  constexpr int V = 4;
+  const int t0 = blockIdx.x * TB;
+  const int c = V * (blockIdx.y * blockDim.x + threadIdx.x);
+  if (c >= C) return;
+  float wt[V * TAPS], in[TB][V], hist[TAPS > 1 ? TAPS - 1 : 1][V], b0[V];
+#pragma unroll
+  for (int j = 0; j < TAPS; j++) LdV<float, V>::ld(w + (int64_t)c * TAPS + V * j, wt + V * j);
+#pragma unroll
+  for (int k = 0; k < TB; k++)
+    if (t0 + k < T) LdV<E, V>::ld(u + (int64_t)(t0 + k) * u_ld + c, in[k]);
+#pragma unroll
+  for (int q = 0; q < V; q++) b0[q] = 0.f;
+  if (bias) LdV<float, V>::ld(bias + c, b0);
+#pragma unroll
+  for (int k = 0; k < TB; k++) {
+    const int t = t0 + k;
+    if (t >= T) break;
+    const int b = seq_of[t], i = t - cu[b];
+    if (k == 0 || i == 0) {                                         // the inputs before this token, from memory
+      const int64_t p = pos[t];
+      const float* st = state + (int64_t)slots[b] * (TAPS - 1) * C + c;
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; j++) {
+        const int back = TAPS - 1 - j;
+#pragma unroll
+        for (int q = 0; q < V; q++) hist[j][q] = 0.f;
+        if (back <= i) LdV<E, V>::ld(u + (int64_t)(t - back) * u_ld + c, hist[j]);
+        else if (p - back >= 0) LdV<float, V>::ld(st + (int64_t)(TAPS - 1 + i - back) * C, hist[j]);
+      }
+    }
+    float acc[V];
+#pragma unroll
+    for (int q = 0; q < V; q++) {
+      acc[q] = b0[q];
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; j++) acc[q] = fmaf(wt[q * TAPS + j], hist[j][q], acc[q]);
+      acc[q] = fmaf(wt[q * TAPS + TAPS - 1], in[k][q], acc[q]);
+      if (ACT) acc[q] = silu(acc[q]);
+    }
+    stv<V>(out + (int64_t)t * C + c, acc);
+#pragma unroll
+    for (int q = 0; q < V; q++) {
+#pragma unroll
+      for (int j = 0; j + 1 < TAPS - 1; j++) hist[j][q] = hist[j + 1][q];
+      if (TAPS > 1) hist[TAPS > 1 ? TAPS - 2 : 0][q] = in[k][q];
+    }
+  }
+}
+
 // after a portion of n tokens that started at position p0: the slot holds the inputs of positions p0 + n - taps + 1 ..
 // p0 + n - 1 (zeros for positions before 0)
 template <typename E>
@@ -314,6 +372,29 @@ void conv_silu(bool bf16, const void* u, int64_t u_ld, const float* w, const flo
   const bool v4 = (C & 3) == 0 && (u_ld & 3) == 0 && ((uintptr_t)u % (4 * eb)) == 0;
   const int cw = v4 ? C / 4 : C;
   dim3 grid(T, (cw + 255) / 256), gs(B, (C + 255) / 256);
+  if (v4 && !single && T >= 64 && taps <= 4 && (uintptr_t)w % 16 == 0 && (!b || (uintptr_t)b % 16 == 0)) {
+    const dim3 gb((T + TB - 1) / TB, (cw + 255) / 256);
+#define SSM_BLOCK(E, TP)                                                                                             \
+  if (act)                                                                                                           \
+    conv_block_k<E, TP, true><<<gb, 256, 0, st>>>((const E*)u, u_ld, w, b, state, cu, seq_of, slots, pos, out, T, C); \
+  else                                                                                                               \
+    conv_block_k<E, TP, false><<<gb, 256, 0, st>>>((const E*)u, u_ld, w, b, state, cu, seq_of, slots, pos, out, T, C)
+#define SSM_TAPS(E)                        \
+  switch (taps) {                          \
+    case 1: SSM_BLOCK(E, 1); break;        \
+    case 2: SSM_BLOCK(E, 2); break;        \
+    case 3: SSM_BLOCK(E, 3); break;        \
+    default: SSM_BLOCK(E, 4);              \
+  }
+    if (bf16) { SSM_TAPS(__bf16) } else { SSM_TAPS(float) }
+#undef SSM_TAPS
+#undef SSM_BLOCK
+    if (taps > 1) {
+      if (bf16) conv_state_k<__bf16><<<gs, 256, 0, st>>>((const __bf16*)u, u_ld, taps, state, cu, slots, pos, C);
+      else conv_state_k<float><<<gs, 256, 0, st>>>((const float*)u, u_ld, taps, state, cu, slots, pos, C);
+    }
+    return;
+  }
 #define SSM_CONV(E, V)                                                                                               \
   if (act)                                                                                                           \
     conv_silu_k<E, V, true><<<grid, 256, 0, st>>>((const E*)u, u_ld, w, b, taps, state, cu, seq_of, slots, pos, out, \

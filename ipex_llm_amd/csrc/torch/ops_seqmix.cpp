@@ -78,12 +78,12 @@ void check_table(const Tensor& table, const char* who) {
 
 void sm_rope_rows_(Tensor& q, int64_t offset, const Tensor& table, const Tensor& pos) {
   c10::DeviceGuard g(q.device());
-  TORCH_CHECK(q.is_cuda() && q.dim() == 3 && is_act(q) && q.is_contiguous(), "sm_rope_rows_: q [T, H, D] contiguous");
+  TORCH_CHECK(q.is_cuda() && q.dim() == 3 && is_act(q) && q.stride(2) == 1, "sm_rope_rows_: q [T, H, D] (unit inner stride)");
   check_table(table, "sm_rope_rows_");
   const int64_t T = q.size(0), H = q.size(1), Dh = q.size(2), dims = 2 * table.size(1);
   TORCH_CHECK(offset >= 0 && offset + dims <= Dh, "sm_rope_rows_: rotated range outside the head");
   check_idx(pos, at::kLong, T, "sm_rope_rows_: pos int64 [T]");
-  illm::sm::rope_rows(bf(q), q.data_ptr(), (int)T, (int)H, (int)Dh, (int)offset, table.data_ptr<float>(),
+  illm::sm::rope_rows(bf(q), q.data_ptr(), q.stride(0), q.stride(1), (int)T, (int)H, (int)offset, table.data_ptr<float>(),
                       (int)table.size(0), (int)dims, pos.data_ptr<int64_t>(), stream());
 }
 
@@ -162,11 +162,23 @@ Tensor sm_latent_attention(const Tensor& q_lat, const Tensor& q_rot, const Tenso
               "sm_latent_attention: a key tile of r + dr = ", r + dr, " does not fit in LDS");
   Tensor out = at::empty({T, H, r}, q_lat.options());
   if (T == 0) return out;
+  auto a16 = [](const Tensor& x) { return (uintptr_t)x.data_ptr() % 16 == 0; };
+  const bool wide = bf(q_lat) && illm::sm::latent_decode_fits((int)r, (int)dr) && a16(q_lat) && a16(rows) &&
+                    (dr == 0 || (a16(q_rot) && q_rot.stride(0) % 8 == 0 && q_rot.stride(1) % 8 == 0));
   // a window spans at most window keys plus the rest of its first tile
   const int64_t span = window > 0 ? std::min<int64_t>(max_ctx, window + 64) : max_ctx;
-  const int nsplit = illm::sm::latent_attention_splits(bf(q_lat), (int)T, (int)H, (int)r, (int)dr, (int)span);
+  const int nsplit = wide ? illm::sm::latent_decode_splits((int)T, (int)H, (int)span)
+                          : illm::sm::latent_attention_splits(bf(q_lat), (int)T, (int)H, (int)r, (int)dr, (int)span);
   Tensor part;
   if (nsplit > 1) part = at::empty({T, H, nsplit, r + 2}, q_lat.options().dtype(at::kFloat));
+  if (wide) {
+    illm::sm::latent_decode(q_lat.data_ptr(), q_rot.data_ptr(), q_rot.stride(0), q_rot.stride(1), rows.data_ptr(),
+                            (int)rows.size(1), block_tables.data_ptr<int32_t>(), (int)block_tables.size(1),
+                            seq_of.data_ptr<int32_t>(), pos.data_ptr<int64_t>(), (float)scale, gp, gst, sp, out.data_ptr(),
+                            nsplit > 1 ? part.data_ptr<float>() : nullptr, nsplit, (int)T, (int)H, (int)r, (int)dr,
+                            (int)window, stream());
+    return out;
+  }
   illm::sm::latent_attention(bf(q_lat), q_lat.data_ptr(), q_rot.data_ptr(), q_rot.stride(0), q_rot.stride(1),
                              rows.data_ptr(), (int)rows.size(1), block_tables.data_ptr<int32_t>(),
                              (int)block_tables.size(1), seq_of.data_ptr<int32_t>(), pos.data_ptr<int64_t>(), (float)scale,
@@ -175,8 +187,24 @@ Tensor sm_latent_attention(const Tensor& q_lat, const Tensor& q_rot, const Tenso
   return out;
 }
 
-// scores f32 [R, L] (R = tokens x H rows) -> causal softmax weights; bf16 pair (hi, lo) or in place (f32)
-std::tuple<Tensor, Tensor> sm_causal_softmax(Tensor& scores, const Tensor& pos, int64_t H, double scale, bool act_f32,
+// x [M, H, K] (strided view) and w [H, N, K], 16-bit, at most 16 rows -> [M, H, N]
+Tensor sm_head_linear(const Tensor& x, const Tensor& w) {
+  c10::DeviceGuard g(x.device());
+  TORCH_CHECK(x.is_cuda() && x.dim() == 3 && bf(x) && w.is_cuda() && w.dim() == 3 && bf(w) && w.is_contiguous(),
+              "sm_head_linear: 16-bit x [M, H, K], w [H, N, K]");
+  const int64_t M = x.size(0), H = x.size(1), K = x.size(2), N = w.size(1);
+  TORCH_CHECK(M <= 16 && K % 32 == 0 && w.size(0) == H && w.size(2) == K && x.stride(2) == 1 && x.stride(0) % 8 == 0 &&
+                  x.stride(1) % 8 == 0 && (uintptr_t)x.data_ptr() % 16 == 0 && (uintptr_t)w.data_ptr() % 16 == 0 && H <= 65535,
+              "sm_head_linear: at most 16 rows, K a multiple of 32, 16-byte aligned rows");
+  Tensor out = at::empty({M, H, N}, x.options());
+  illm::sm::head_linear(x.data_ptr(), x.stride(0), x.stride(1), (int)M, (int)H, (int)K, w.data_ptr(), (int)N, out.data_ptr(),
+                        stream());
+  return out;
+}
+
+// scores f32 [R, L] (R = tokens x H rows) -> causal softmax weights; bf16 pairs [R, 2 L] (hi halves, then lo halves) or
+// in place (f32)
+Tensor sm_causal_softmax(Tensor& scores, const Tensor& pos, int64_t H, double scale, bool act_f32,
                                              int64_t key0, int64_t window, const c10::optional<Tensor>& sink) {
   c10::DeviceGuard g(scores.device());
   TORCH_CHECK(scores.is_cuda() && scores.dim() == 2 && scores.scalar_type() == at::kFloat && scores.is_contiguous(),
@@ -185,16 +213,12 @@ std::tuple<Tensor, Tensor> sm_causal_softmax(Tensor& scores, const Tensor& pos, 
   TORCH_CHECK(H >= 1 && R % H == 0, "sm_causal_softmax: rows must be tokens x heads");
   TORCH_CHECK(key0 >= 0 && window >= 0 && window < (int64_t)1 << 30, "sm_causal_softmax: key0 >= 0, window >= 0");
   check_idx(pos, at::kLong, R / H, "sm_causal_softmax: pos int64 [R / H]");
-  Tensor hi, lo;
-  if (!act_f32) {
-    hi = at::empty({R, L}, scores.options().dtype(at::kBFloat16));
-    lo = at::empty({R, L}, scores.options().dtype(at::kBFloat16));
-  }
-  illm::sm::causal_softmax(!act_f32, scores.data_ptr<float>(), L, pos.data_ptr<int64_t>(), (int)H, (float)scale, R, (int)L,
-                           act_f32 ? nullptr : hi.data_ptr(), act_f32 ? nullptr : lo.data_ptr(), key0, (int)window,
-                           sink_ptr(sink, H, "sm_causal_softmax"), stream());
-  if (act_f32) return {scores, scores};
-  return {hi, lo};
+  Tensor hl;
+  if (!act_f32) hl = at::empty({R, 2 * L}, scores.options().dtype(at::kBFloat16));
+  illm::sm::causal_softmax(!act_f32, scores.data_ptr<float>(), pos.data_ptr<int64_t>(), (int)H, (float)scale, R, (int)L,
+                           act_f32 ? nullptr : hl.data_ptr(), key0, (int)window, sink_ptr(sink, H, "sm_causal_softmax"),
+                           stream());
+  return act_f32 ? scores : hl;
 }
 
 Tensor sm_mlstm_scan(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& ipre, const Tensor& fpre,
@@ -285,11 +309,12 @@ TORCH_LIBRARY_FRAGMENT(ipex_llm_amd, m) {
         "Tensor(a!) rows) -> ()");
   m.def("sm_latent_attention(Tensor q_lat, Tensor q_rot, Tensor rows, Tensor block_tables, Tensor seq_of, Tensor pos, "
         "float scale, Tensor? gate, int max_ctx, bool act_f32, int window=0, Tensor? sink=None) -> Tensor");
+  m.def("sm_head_linear(Tensor x, Tensor w) -> Tensor");
   m.def("sm_latent_attention_fits(bool bf16, int H, int r, int dr) -> int");
   m.def("sm_mlstm_scan(Tensor q, Tensor k, Tensor v, Tensor ipre, Tensor fpre, Tensor ib, Tensor fb, float cap, "
         "Tensor(a!) S, Tensor(b!) n, Tensor(c!) m, Tensor cu, Tensor slots, Tensor pos, int max_q) -> Tensor");
   m.def("sm_causal_softmax(Tensor(a!) scores, Tensor pos, int H, float scale, bool act_f32, int key0=0, int window=0, "
-        "Tensor? sink=None) -> (Tensor, Tensor)");
+        "Tensor? sink=None) -> Tensor");
   m.def("sm_head_rms_gate(Tensor h, Tensor norm_w, Tensor gate, float eps, bool act_f32, bool silu=False) -> Tensor");
   m.def("sm_glu_gelu(Tensor gu) -> Tensor");
   m.def("sm_glu_act(Tensor gu, int act) -> Tensor");
@@ -308,6 +333,7 @@ TORCH_LIBRARY_IMPL(ipex_llm_amd, CUDA, m) {
   m.impl("sm_latent_attention", &sm_latent_attention);
   m.impl("sm_mlstm_scan", &sm_mlstm_scan);
   m.impl("sm_causal_softmax", &sm_causal_softmax);
+  m.impl("sm_head_linear", &sm_head_linear);
   m.impl("sm_head_rms_gate", &sm_head_rms_gate);
   m.impl("sm_glu_gelu", &sm_glu_gelu);
   m.impl("sm_glu_act", &sm_glu_act);

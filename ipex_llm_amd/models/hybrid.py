@@ -404,6 +404,9 @@ class LatentAttention(nn.Module):
         self.dkv_norm = nn.Parameter(dkv_norm, requires_grad=False)
         self.w_uk = nn.Parameter(w_uk.view(H, s.dim, r).contiguous(), requires_grad=False)               # [H, dim, r]
         self.w_uv_t = nn.Parameter(w_uv.view(H, s.vdim, r).transpose(1, 2).contiguous(), requires_grad=False)  # [H, r, dv]
+        # the same two in the other order, for the decode-size kernel
+        self.w_uk_t = nn.Parameter(w_uk.view(H, s.dim, r).transpose(1, 2).contiguous(), requires_grad=False)  # [H, r, dim]
+        self.w_uv = nn.Parameter(w_uv.view(H, s.vdim, r).contiguous(), requires_grad=False)              # [H, dv, r]
         self.sink = nn.Parameter(sink.float().contiguous(), requires_grad=False) if s.sink else None
         self.w_o = nn.Parameter(w_o, requires_grad=False)
         self.table: Optional[torch.Tensor] = None
@@ -421,7 +424,7 @@ class LatentAttention(nn.Module):
         s = self.s
         T, H = xa.shape[0], s.heads
         y = BM.linear(xa, self.w_in)
-        q = y[:, :self.n_q].reshape(T, H, s.dim + s.rot_dim).contiguous()
+        q = y[:, :self.n_q].view(T, H, s.dim + s.rot_dim)
         dkv = y[:, self.n_q:self.n_q + self.n_dkv]
         gate = y[:, self.n_q + self.n_dkv:] if s.out_gate else None
         head_gate = gate if s.gate == "head" else None
@@ -429,11 +432,11 @@ class LatentAttention(nn.Module):
         SM.latent_kv_store(dkv, self.dkv_norm, eps, s.kv_rank, table, pos, slots, cache.rows[li])
         SM.rope_rows_(q, s.dim, table, pos)
         # absorbed up-projection of the keys: per-head [T, dim] x [dim, r]
-        q_lat = torch.bmm(q[..., :s.dim].transpose(0, 1), self.w_uk).transpose(0, 1)
+        q_lat = SM.head_linear(q[..., :s.dim], self.w_uk, self.w_uk_t)
         o_lat = SM.latent_attention(q_lat, q[..., s.dim:], cache.rows[li], meta.block_tables, meta.seq_of, pos,
                                     s.scale, head_gate, meta.q_lens_host, meta.seq_lens_host, xa.dtype,
                                     window=s.window, sink=self.sink)
-        o = torch.bmm(o_lat.transpose(0, 1), self.w_uv_t).transpose(0, 1).reshape(T, H * s.vdim)
+        o = SM.head_linear(o_lat, self.w_uv_t, self.w_uv).reshape(T, H * s.vdim)
         if gate is not None and s.gate == "element":
             o = MA.sigmoid_gate(o, gate)
         return BM.linear(o, self.w_o)
@@ -931,7 +934,7 @@ class ChannelDelta(nn.Module):
         g = CX.lowrank_decay(a1, self.w_a2, self.rate, self.dt_bias, "softplus").view(T, H, d)
         o = CX.channel_delta_scan(q, k, v, g, b, d ** -0.5, st["chan_delta"], meta.cu_q, meta.state_slots, pos,
                                   meta.q_lens_host)
-        gate = BM.linear(g1.contiguous(), self.w_g2)
+        gate = BM.linear(g1, self.w_g2)
         return BM.linear(SM.head_rms_gate(o, self.norm, gate, eps, y.dtype), self.w_o)
 
 

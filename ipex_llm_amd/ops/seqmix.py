@@ -24,7 +24,7 @@ import torch
 import torch.nn.functional as F
 
 __all__ = ["embed_bigram", "add_scaled_layer_norm_", "layer_norm_f32", "latent_kv_store", "rope_rows_",
-           "latent_attention", "mlstm_scan", "head_rms_gate", "glu_gelu", "glu_act", "GLU_ACTS", "rope_table", "native"]
+           "head_linear", "latent_attention", "mlstm_scan", "head_rms_gate", "glu_gelu", "glu_act", "GLU_ACTS", "rope_table", "native"]
 
 
 def native(t: torch.Tensor) -> bool:
@@ -155,6 +155,17 @@ def latent_kv_store(dkv: torch.Tensor, norm_w: torch.Tensor, eps: float, rank: i
 
 
 # ------------------------------------------------------------------ latent attention
+def head_linear(x: torch.Tensor, w_kn: torch.Tensor, w_nk: torch.Tensor) -> torch.Tensor:
+    """``x[:, h] @ w_kn[h]`` for every head: ``x`` [T, H, K] (a strided view is allowed), ``w_kn`` [H, K, N] and
+    ``w_nk`` [H, N, K] the same matrices in both orders.  Decode-size steps (at most 16 rows, 16-bit) run one kernel
+    over ``w_nk``, others a batched library product over ``w_kn``.  Returns [T, H, N] (a strided view)."""
+    T, K = x.shape[0], x.shape[2]
+    if x.is_cuda and T <= 16 and x.dtype == torch.bfloat16 and K % 32 == 0 and x.stride(2) == 1 and \
+            x.stride(0) % 8 == 0 and x.stride(1) % 8 == 0 and x.data_ptr() % 16 == 0 and native(x):
+        return _ops().sm_head_linear(x, w_nk)
+    return torch.bmm(x.transpose(0, 1), w_kn).transpose(0, 1)
+
+
 def latent_attention(q_lat: torch.Tensor, q_rot: torch.Tensor, rows: torch.Tensor, block_tables: torch.Tensor,
                      seq_of: torch.Tensor, pos: torch.Tensor, scale: float, gate: Optional[torch.Tensor],
                      q_lens: List[int], ctx_lens: List[int], out_dtype: torch.dtype, window: int = 0,
@@ -225,14 +236,13 @@ def _mm_f32(a: torch.Tensor, b: torch.Tensor) -> torch.Tensor:
     return a.float() @ b.float()
 
 
-def _latent_attention_gemm(q_lat, q_rot, rows, table_row, pos, scale, L: int, n: int, window: int = 0,
-                           sink=None) -> torch.Tensor:
-    """one sequence's portion of n >= GEMM_MIN_Q tokens ending at key count L -> f32 [n, H, r]"""
+def _latent_attention_gemm(q_lat, q_rot, rows, table_row, pos, scale, gate, L: int, n: int, out: torch.Tensor,
+                           window: int = 0, sink=None) -> None:
+    """one sequence's portion of n >= GEMM_MIN_Q tokens ending at key count L -> ``out`` [n, H, r]"""
     _, H, r = q_lat.shape
     bs = rows.shape[1]
     nb = (L + bs - 1) // bs
     kv = rows[table_row[:nb].long()].reshape(nb * bs, -1)           # this sequence's rows, in order
-    out = torch.empty(n, H, r, dtype=torch.float32, device=q_lat.device)
     f32 = q_lat.dtype == torch.float32
     for t0 in range(0, n, GEMM_Q_BLOCK):
         t1 = min(n, t0 + GEMM_Q_BLOCK)
@@ -240,13 +250,11 @@ def _latent_attention_gemm(q_lat, q_rot, rows, table_row, pos, scale, L: int, n:
         k0 = max(0, L - n + t0 - window + 1) // 8 * 8 if window > 0 else 0      # the first key its first token sees
         q2 = torch.cat([q_lat[t0:t1], q_rot[t0:t1]], -1).reshape((t1 - t0) * H, -1)
         sc = _mm_f32(q2, kv[k0:Lb].t()).contiguous()
-        hi, lo = _ops().sm_causal_softmax(sc, pos[t0:t1].contiguous(), H, scale, f32, k0, window, sink)
+        w = _ops().sm_causal_softmax(sc, pos[t0:t1].contiguous(), H, scale, f32, k0, window, sink)
         c = kv[k0:Lb, :r]
-        o = _mm_f32(hi, c)
-        if not f32:
-            o += _mm_f32(lo, c)
-        out[t0:t1] = o.view(t1 - t0, H, r)
-    return out
+        # f32 weights against 16-bit latents: hi + lo halves side by side along the summed axis, the latents twice
+        o = _mm_f32(w, c if f32 else torch.cat([c, c], 0)).view(t1 - t0, H, r)
+        out[t0:t1] = o if gate is None else o * torch.sigmoid(gate[t0:t1].float())[..., None]
 
 
 def _latent_attention_gpu(q_lat, q_rot, rows, block_tables, seq_of, pos, scale, gate, q_lens, ctx_lens, out_dtype,
@@ -263,11 +271,8 @@ def _latent_attention_gpu(q_lat, q_rot, rows, block_tables, seq_of, pos, scale, 
     small, small_ctx, t0 = [], 1, 0
     for b, (n, L) in enumerate(zip(q_lens, ctx_lens)):
         if n >= min_q:
-            o = _latent_attention_gemm(q_lat[t0:t0 + n], q_rot[t0:t0 + n], rows, block_tables[b], pos[t0:t0 + n], scale,
-                                       L, n, window, sink)
-            if gate is not None:
-                o = o * torch.sigmoid(gate[t0:t0 + n].float())[..., None]
-            out[t0:t0 + n] = o.to(out_dtype)
+            _latent_attention_gemm(q_lat[t0:t0 + n], q_rot[t0:t0 + n], rows, block_tables[b], pos[t0:t0 + n], scale,
+                                   gate[t0:t0 + n] if gate is not None else None, L, n, out[t0:t0 + n], window, sink)
         elif n:
             small.append(torch.arange(t0, t0 + n, device=q_lat.device))
             small_ctx = max(small_ctx, L)
