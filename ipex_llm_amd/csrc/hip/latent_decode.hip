@@ -24,6 +24,7 @@ typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
 typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
+typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 
 constexpr int KT = 64;                                              // keys per tile
 constexpr int PF = 18;                                              // 16-byte pieces of a tile per thread (D <= 576)
@@ -70,15 +71,14 @@ __global__ void __launch_bounds__(256) latent_dec_k(const __bf16* __restrict__ q
   const int32_t* tab = bt + (int64_t)seq_of[t] * bt_w;
   const int ntiles = (int)(p / KT) + 1;
   const int64_t lo = window > 0 ? (p - window + 1 > 0 ? p - window + 1 : 0) : 0;
-  uint4 pf[PF];
-  int n8 = 0;                                                       // pieces of the requested tile
+  u32x4 pf[PF];
+  const int krow = tid >> 2, kpc = tid & 3;                         // four threads per key: pieces kpc, kpc + 4, ...
   auto request = [&](int ti) {
     const int64_t k0 = (int64_t)ti * KT;
-    n8 = (int)min((int64_t)KT, p - k0 + 1) * D8;
-    const uint4* src = (const uint4*)(rows + ((int64_t)tab[k0 / bs] * bs + (k0 % bs)) * D);
+    const int row = min(krow, (int)min((int64_t)KT, p - k0 + 1) - 1);          // (past the last key: that one again)
+    const u32x4* src = (const u32x4*)(rows + ((int64_t)tab[k0 / bs] * bs + (k0 % bs) + row) * D);
 #pragma unroll
-    for (int u = 0; u < PF; u++)
-      if (tid + 256 * u < n8) pf[u] = src[tid + 256 * u];
+    for (int u = 0; u < PF; u++) pf[u] = src[min(kpc + 4 * u, D8 - 1)];
   };
   int ti = (int)(lo / KT) + zs;
   if (ti < ntiles) request(ti);
@@ -102,15 +102,10 @@ __global__ void __launch_bounds__(256) latent_dec_k(const __bf16* __restrict__ q
   for (; ti < ntiles; ti += nsplit) {
     const int64_t k0 = (int64_t)ti * KT;
     const int nvalid = (int)min((int64_t)KT, p - k0 + 1);
-    {
-      int j = 0, c = 8 * tid;
-      while (c >= D) { c -= D; j++; }
+    if (krow < nvalid) {
 #pragma unroll
-      for (int u = 0; u < PF; u++) {
-        if (tid + 256 * u < n8) *(uint4*)(kt + j * DP + c) = pf[u];
-        c += 8 * 256;
-        while (c >= D) { c -= D; j++; }
-      }
+      for (int u = 0; u < PF; u++)
+        if (kpc + 4 * u < D8) *(u32x4*)(kt + krow * DP + 8 * (kpc + 4 * u)) = pf[u];
     }
     __syncthreads();
     if (ti + nsplit < ntiles) request(ti + nsplit);

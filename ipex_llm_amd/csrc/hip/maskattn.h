@@ -51,6 +51,13 @@ void chunk_softmax(bool bf16, float* sc, int64_t R, int Lq, int L, int G, int re
 void talk_mix(bool bf16, const float* w, const float* talk, int64_t pieces, int Lq, int L, int G, int rep, void* hl,
               float* out32, hipStream_t st);
 
+// a block of nq queries (rows of q f32 [T, H, d] from tok0 on) and the keys it sees (positions 0 .. nkeep - 1, then nr from k0
+// on, padded to nk columns) as operands of batched products per key head: 16-bit rows: q2 [G, nq rep, 2 d] (hi and lo halves),
+// k2 [G, 2 d, nk], v2 [G, 2 nk, dv] (everything twice); f32 rows: once.  tab: the sequence's row of the block table
+void pack_block(bool bf16, const float* q, int64_t tok0, int nq, const void* rows, int bs, const int32_t* tab, int nkeep,
+                int64_t k0, int nr, int nk, void* q2, void* k2, void* v2, int H, int G, int d, int dv, hipStream_t st);
+// o f32 [G, nq rep, dv] -> rows tok0 .. of out [T, H dv] in the activation type
+void unpack_block(bool bf16, const float* o, void* out, int64_t tok0, int nq, int H, int G, int dv, hipStream_t st);
 // o[t, c] *= sigmoid(g[t, c]); g rows of g_ld elements
 void sigmoid_gate(bool bf16, void* o, const void* g, int64_t g_ld, int64_t T, int C, int per, hipStream_t st);
 

@@ -676,6 +676,76 @@ __global__ void __launch_bounds__(256) chunk_softmax_k(float* __restrict__ sc, i
   }
 }
 
+// ------------------------------------------------------------------ operands of the batched products
+// a block of queries and the keys it sees as operands of two batched products per key head.  16-bit rows: f32 queries as hi
+// and lo halves side by side along the summed axis, so keys (and values, for f32 weights) appear twice
+template <typename E>
+__global__ void __launch_bounds__(256) pack_queries_k(const float* __restrict__ q, int64_t tok0, int nq, E* __restrict__ q2,
+                                                     int H, int G, int d) {
+  const int rep = H / G, tok = blockIdx.x;
+  constexpr int TW = sizeof(E) == 2 ? 2 : 1;
+  for (int i = threadIdx.x; i < H * d; i += blockDim.x) {
+    const int h = i / d, c = i - h * d, g = h / rep;
+    const float v = q[(tok0 + tok) * H * d + i];
+    E* o = q2 + (((int64_t)g * nq + tok) * rep + (h - g * rep)) * TW * d;
+    const E hi = (E)v;
+    o[c] = hi;
+    if (TW == 2) o[d + c] = (E)(v - (float)hi);
+  }
+}
+
+// column j: position j below nkeep, then k0, k0 + 1, ... (past the last key: that one again).  k2 [G, TW d, nk], v2 [G, TW nk,
+// dv]; a workgroup per 64 columns of a key head, the keys turned through LDS
+template <typename E>
+__global__ void __launch_bounds__(256) pack_keys_k(const E* __restrict__ rows, int bs, const int32_t* __restrict__ tab,
+                                                  int nkeep, int64_t k0, int nr, int nk, E* __restrict__ k2,
+                                                  E* __restrict__ v2, int G, int d, int dv) {
+  constexpr int TW = sizeof(E) == 2 ? 2 : 1;
+  __shared__ E tile[64][65];
+  __shared__ int64_t at[64];
+  const int j0 = blockIdx.x * 64, g = blockIdx.y, nj = min(64, nk - j0);
+  const int64_t ld = (int64_t)G * (d + dv);
+  if (threadIdx.x < 64) {
+    const int j = min(j0 + (int)threadIdx.x, nk - 1);
+    const int64_t p = j < nkeep ? j : k0 + min(j - nkeep, nr - 1);
+    at[threadIdx.x] = ((int64_t)tab[p / bs] * bs + p % bs) * ld;
+  }
+  __syncthreads();
+  for (int c0 = 0; c0 < d; c0 += 64) {
+    const int nc = min(64, d - c0);
+    __syncthreads();
+    for (int i = threadIdx.x; i < 64 * 64; i += 256) {
+      const int j = i >> 6, c = i & 63;
+      if (j < nj && c < nc) tile[j][c] = rows[at[j] + (int64_t)g * d + c0 + c];
+    }
+    __syncthreads();
+    for (int i = threadIdx.x; i < 64 * 64; i += 256) {
+      const int c = i >> 6, j = i & 63;
+      if (j < nj && c < nc) {
+#pragma unroll
+        for (int w = 0; w < TW; w++) k2[((int64_t)g * TW * d + w * d + c0 + c) * nk + j0 + j] = tile[j][c];
+      }
+    }
+  }
+  for (int i = threadIdx.x; i < nj * dv; i += 256) {
+    const int j = i / dv, c = i - j * dv;
+    const E v = rows[at[j] + (int64_t)G * d + (int64_t)g * dv + c];
+#pragma unroll
+    for (int w = 0; w < TW; w++) v2[((int64_t)g * TW * nk + (int64_t)w * nk + j0 + j) * dv + c] = v;
+  }
+}
+
+// o [G, nq, rep, dv] -> out[tok0 + tok] = [heads in order]
+template <typename E>
+__global__ void __launch_bounds__(256) unpack_k(const float* __restrict__ o, E* __restrict__ out, int64_t tok0, int nq, int H,
+                                               int G, int dv) {
+  const int rep = H / G, tok = blockIdx.x;
+  for (int i = threadIdx.x; i < H * dv; i += blockDim.x) {
+    const int h = i / dv, c = i - h * dv, g = h / rep;
+    stf(out + (tok0 + tok) * H * dv + i, o[(((int64_t)g * nq + tok) * rep + (h - g * rep)) * dv + c]);
+  }
+}
+
 // per: consecutive values that share a gate.  V values per thread (V = 8: 16-byte accesses; C, and per unless it is 1,
 // are multiples of 8)
 template <typename E, int V>
@@ -851,6 +921,23 @@ void chunk_softmax(bool bf16, float* sc, int64_t R, int Lq, int L, int G, int re
     if (bf16) MA_SOFT(__bf16, 0); else MA_SOFT(float, 0);
   }
 #undef MA_SOFT
+}
+
+void pack_block(bool bf16, const float* q, int64_t tok0, int nq, const void* rows, int bs, const int32_t* tab, int nkeep,
+                int64_t k0, int nr, int nk, void* q2, void* k2, void* v2, int H, int G, int d, int dv, hipStream_t st) {
+  if (nq <= 0 || nk <= 0) return;
+  const dim3 gk((nk + 63) / 64, G);
+#define MA_PACK(E)                                                                                                  \
+  pack_queries_k<E><<<nq, 256, 0, st>>>(q, tok0, nq, (E*)q2, H, G, d);                                              \
+  pack_keys_k<E><<<gk, 256, 0, st>>>((const E*)rows, bs, tab, nkeep, k0, nr, nk, (E*)k2, (E*)v2, G, d, dv)
+  if (bf16) { MA_PACK(__bf16); } else { MA_PACK(float); }
+#undef MA_PACK
+}
+
+void unpack_block(bool bf16, const float* o, void* out, int64_t tok0, int nq, int H, int G, int dv, hipStream_t st) {
+  if (nq <= 0) return;
+  if (bf16) unpack_k<__bf16><<<nq, 256, 0, st>>>(o, (__bf16*)out, tok0, nq, H, G, dv);
+  else unpack_k<float><<<nq, 256, 0, st>>>(o, (float*)out, tok0, nq, H, G, dv);
 }
 
 void talk_mix(bool bf16, const float* w, const float* talk, int64_t pieces, int Lq, int L, int G, int rep, void* hl,

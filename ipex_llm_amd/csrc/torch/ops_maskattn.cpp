@@ -191,6 +191,42 @@ Tensor ma_talk_mix(const Tensor& w, const Tensor& talk, int64_t Lq, int64_t G, i
   return out;
 }
 
+std::tuple<Tensor, Tensor, Tensor> ma_pack_block(const Tensor& q, int64_t tok0, int64_t nq, const Tensor& rows,
+                                                 const Tensor& table_row, int64_t G, int64_t dv, int64_t nkeep, int64_t k0,
+                                                 int64_t nr, int64_t nk) {
+  c10::DeviceGuard g(q.device());
+  TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.scalar_type() == at::kFloat && q.is_contiguous() && tok0 >= 0 && nq >= 1 &&
+                  tok0 + nq <= q.size(0),
+              "ma_pack_block: queries f32 [T, H, d] contiguous, the block inside them");
+  const int64_t H = q.size(1), d = q.size(2);
+  const auto ty = rows.scalar_type();
+  TORCH_CHECK(rows.is_cuda() && rows.dim() == 3 && rows.is_contiguous() && (ty == at::kBFloat16 || ty == at::kFloat) &&
+                  G >= 1 && H % G == 0 && dv >= 1 && rows.size(2) == G * (d + dv) && G <= 65535,
+              "ma_pack_block: rows [blocks, bs, G (d + dv)]");
+  TORCH_CHECK(table_row.is_cuda() && table_row.dim() == 1 && table_row.scalar_type() == at::kInt && table_row.is_contiguous() &&
+                  nkeep >= 0 && k0 >= nkeep && nr >= 1 && nk >= nkeep + nr && k0 + nr <= table_row.size(0) * rows.size(1),
+              "ma_pack_block: block table row int32, the keys inside it");
+  const int64_t tw = ty == at::kBFloat16 ? 2 : 1;
+  Tensor q2 = at::empty({G, nq * (H / G), tw * d}, rows.options()), k2 = at::empty({G, tw * d, nk}, rows.options()),
+         v2 = at::empty({G, tw * nk, dv}, rows.options());
+  illm::ma::pack_block(tw == 2, q.data_ptr<float>(), tok0, (int)nq, rows.data_ptr(), (int)rows.size(1),
+                       table_row.data_ptr<int32_t>(), (int)nkeep, k0, (int)nr, (int)nk, q2.data_ptr(), k2.data_ptr(),
+                       v2.data_ptr(), (int)H, (int)G, (int)d, (int)dv, stream());
+  return {q2, k2, v2};
+}
+
+void ma_unpack_block(const Tensor& o, Tensor& out, int64_t tok0, int64_t nq, int64_t H) {
+  c10::DeviceGuard g(o.device());
+  TORCH_CHECK(o.is_cuda() && o.dim() == 3 && o.scalar_type() == at::kFloat && o.is_contiguous() && H >= 1 &&
+                  H % o.size(0) == 0 && o.size(1) == nq * (H / o.size(0)),
+              "ma_unpack_block: o f32 [G, nq rep, dv] contiguous");
+  TORCH_CHECK(out.is_cuda() && out.dim() == 2 && out.is_contiguous() && out.size(1) == H * o.size(2) && tok0 >= 0 &&
+                  tok0 + nq <= out.size(0) && (out.scalar_type() == at::kBFloat16 || out.scalar_type() == at::kFloat),
+              "ma_unpack_block: out [T, H dv], the block inside it");
+  illm::ma::unpack_block(out.scalar_type() == at::kBFloat16, o.data_ptr<float>(), out.data_ptr(), tok0, (int)nq, (int)H,
+                         (int)o.size(0), (int)o.size(2), stream());
+}
+
 Tensor ma_sigmoid_gate(Tensor& o, const Tensor& gate) {
   c10::DeviceGuard g(o.device());
   TORCH_CHECK(o.is_cuda() && o.dim() == 2 && is_act(o) && o.is_contiguous(), "ma_sigmoid_gate: o [T, C] contiguous");
@@ -213,6 +249,9 @@ TORCH_LIBRARY_FRAGMENT(ipex_llm_amd, m) {
   m.def("ma_masked_attention_fits(bool bf16, int rep, int d, int dv) -> int");
   m.def("ma_chunk_softmax(Tensor(a!) scores, int Lq, int G, int rep, float scale, Tensor? sink, bool act_f32, "
         "float softcap, bool in_place, int window, int keep, int nkeep, int q0, int k0) -> Tensor");
+  m.def("ma_pack_block(Tensor q, int tok0, int nq, Tensor rows, Tensor table_row, int G, int dv, int nkeep, int k0, int nr, "
+        "int nk) -> (Tensor, Tensor, Tensor)");
+  m.def("ma_unpack_block(Tensor o, Tensor(a!) out, int tok0, int nq, int H) -> ()");
   m.def("ma_talk_mix(Tensor w, Tensor talk, int Lq, int G, int rep, bool act_f32) -> Tensor");
   m.def("ma_sigmoid_gate(Tensor(a!) o, Tensor gate) -> Tensor(a!)");
 }
@@ -226,5 +265,7 @@ TORCH_LIBRARY_IMPL(ipex_llm_amd, CUDA, m) {
   m.impl("ma_masked_attention", &ma_masked_attention);
   m.impl("ma_chunk_softmax", &ma_chunk_softmax);
   m.impl("ma_talk_mix", &ma_talk_mix);
+  m.impl("ma_pack_block", &ma_pack_block);
+  m.impl("ma_unpack_block", &ma_unpack_block);
   m.impl("ma_sigmoid_gate", &ma_sigmoid_gate);
 }

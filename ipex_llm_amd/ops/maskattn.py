@@ -217,9 +217,7 @@ def _window_gemm(q, rows, table_row, G, dv, scale, sink, t0, n, L, size, keep, o
     softmax between them."""
     _, H, d = q.shape
     rep = H // G
-    bs = rows.shape[1]
     f32 = rows.dtype == torch.float32
-    flat = rows.view(-1, rows.shape[-1])
     p0 = L - n
     for b0 in range(0, n, WINDOW_Q_BLOCK):
         nq = min(WINDOW_Q_BLOCK, n - b0)
@@ -228,31 +226,16 @@ def _window_gemm(q, rows, table_row, G, dv, scale, sink, t0, n, L, size, keep, o
         nkeep = min(keep, k0)
         nr = q0 + nq - k0
         nk = -(-(nkeep + nr) // 8) * 8                               # padded columns: masked (ahead of every query)
-        p = torch.cat([torch.arange(nkeep, device=q.device), torch.arange(k0, k0 + nr, device=q.device),
-                       torch.full((nk - nkeep - nr,), k0 + nr - 1, device=q.device)])
-        ridx = table_row.long()[p // bs] * bs + p % bs
-        kv = flat.index_select(0, ridx)
-        kk = kv[:, :G * d].reshape(nk, G, d).permute(1, 2, 0)
-        vv = kv[:, G * d:].reshape(nk, G, dv).permute(1, 0, 2)
-        qq = q[t0 + b0:t0 + b0 + nq].view(nq, G, rep, d).permute(1, 0, 2, 3).reshape(G, nq * rep, d)
-        args = (nq, G, rep, scale, sink, f32, softcap)
-        win = (size, keep, nkeep, q0, k0)
-        if f32:
-            sc = torch.bmm(qq, kk)
-            w = _ops().ma_chunk_softmax(sc.view(G * nq * rep, nk), *args, True, *win)
-            if talk is not None:
-                w = _ops().ma_talk_mix(w, talk, nq, G, rep, True)
-            o = torch.bmm(w.view(G, nq * rep, nk), vv)
-        else:
-            qh = qq.to(rows.dtype)
-            q2 = torch.cat([qh, (qq - qh.float()).to(rows.dtype)], -1)
-            sc = torch.bmm(q2, torch.cat([kk, kk], 1), out_dtype=torch.float32)
-            w = _ops().ma_chunk_softmax(sc.view(G * nq * rep, nk), *args, talk is not None, *win)
-            if talk is not None:
-                w = _ops().ma_talk_mix(w, talk, nq, G, rep, False)
-            o = torch.bmm(w.view(G, nq * rep, 2 * nk), torch.cat([vv, vv], 1), out_dtype=torch.float32)
-        o = o.view(G, nq, rep, dv).permute(1, 0, 2, 3).reshape(nq, H * dv)
-        out[t0 + b0:t0 + b0 + nq] = o.to(out.dtype)
+        # 16-bit: f32 queries (and weights) as hi + lo halves side by side along the summed axis, keys and values twice
+        q2, k2, v2 = _ops().ma_pack_block(q, t0 + b0, nq, rows, table_row, G, dv, nkeep, k0, nr, nk)
+        sc = torch.bmm(q2, k2) if f32 else torch.bmm(q2, k2, out_dtype=torch.float32)
+        w = _ops().ma_chunk_softmax(sc.view(G * nq * rep, nk), nq, G, rep, scale, sink, f32, softcap, f32 or talk is not None,
+                                    size, keep, nkeep, q0, k0)
+        if talk is not None:
+            w = _ops().ma_talk_mix(w, talk, nq, G, rep, f32)
+        w = w.view(G, nq * rep, -1)
+        o = torch.bmm(w, v2) if f32 else torch.bmm(w, v2, out_dtype=torch.float32)
+        _ops().ma_unpack_block(o, out, t0 + b0, nq, H)
 
 
 def _masked_attention_gpu(q, rows, G, dv, block_tables, seq_of, pos, scale, mask, size, sink, q_lens, ctx_lens,
