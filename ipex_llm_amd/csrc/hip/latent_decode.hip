@@ -6,9 +6,9 @@
 //                  current one is used.  Every wave scores 16 of the keys against
 //                  all heads on the matrix cores (bf16 as stored, f32
 //                  accumulation); the softmax runs online in f32 over the whole
-//                  tile; the weighted sum is f32 weights x latents on the vector
-//                  unit, a thread owning one or two latent columns of all heads,
-//                  so nothing is merged between waves
+//                  tile; the weighted sum takes the f32 weights as bf16 hi + lo
+//                  halves, every wave owning a quarter of the latent columns of
+//                  all heads, so nothing is merged between waves
 //   combine_k      merge of the key splits with the sink and the head gate
 //   head_linear_k  y[m, h] = x[m, h] W[h]^T for at most 16 rows: the absorbed up-
 //                  projections, a wave per 16 outputs of a head
@@ -21,8 +21,6 @@ namespace sm {
 namespace {
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
-typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
-typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 
@@ -48,7 +46,8 @@ __device__ __forceinline__ float with_sink(float M, float L, const float* sink, 
 
 __host__ __device__ inline int row_of(int D) { return ((D + 31) & ~31) + 8; }
 
-template <int CPT, int HB>
+// NT: 16-column tiles per wave (r <= 64 NT)
+template <int NT>
 __global__ void __launch_bounds__(256) latent_dec_k(const __bf16* __restrict__ q_lat, const __bf16* __restrict__ q_rot,
                                                    int64_t qr_st, int64_t qr_sh, const __bf16* __restrict__ rows, int bs,
                                                    const int32_t* __restrict__ bt, int bt_w,
@@ -58,8 +57,8 @@ __global__ void __launch_bounds__(256) latent_dec_k(const __bf16* __restrict__ q
                                                    float* __restrict__ part, int H, int r, int dr, int window) {
   extern __shared__ __align__(16) unsigned char smem[];
   const int D = r + dr, DP = row_of(D), KS = (D + 31) >> 5, D8 = D >> 3;
-  const int nsplit = gridDim.z, zs = blockIdx.z, t = blockIdx.x, h0 = blockIdx.y * HB;
-  const int nh = min(HB, H - h0);
+  const int nsplit = gridDim.z, zs = blockIdx.z, t = blockIdx.x, h0 = blockIdx.y * 16;
+  const int nh = min(16, H - h0);
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, r16 = lane & 15, g = lane >> 4;
   __bf16* qs = (__bf16*)smem;                                       // [16][DP]
   __bf16* kt = qs + 16 * DP;                                        // [KT][DP]
@@ -92,13 +91,9 @@ __global__ void __launch_bounds__(256) latent_dec_k(const __bf16* __restrict__ q
     *(uint4*)(qs + h * DP + c) = *(const uint4*)s;
   }
   float m_r = -INFINITY, l_r = 0.f;                                 // of head r16, the same in every thread that holds it
-  float o[HB][CPT];
+  f32x4 o[NT];                                                      // heads 4 g + i, column 16 (wv + 4 n) + r16
 #pragma unroll
-  for (int h = 0; h < HB; h++)
-#pragma unroll
-    for (int c = 0; c < CPT; c++) o[h][c] = 0.f;
-  const int c0 = CPT * tid;
-  const bool mine = c0 < r;
+  for (int n = 0; n < NT; n++) o[n] = f32x4{0.f, 0.f, 0.f, 0.f};
   for (; ti < ntiles; ti += nsplit) {
     const int64_t k0 = (int64_t)ti * KT;
     const int nvalid = (int)min((int64_t)KT, p - k0 + 1);
@@ -142,33 +137,33 @@ __global__ void __launch_bounds__(256) latent_dec_k(const __bf16* __restrict__ q
     if (wv == 0 && g == 0) al[r16] = alpha;
     __syncthreads();
     l_r = l_r * alpha + (lred[r16] + lred[16 + r16]) + (lred[32 + r16] + lred[48 + r16]);
-    if (mine) {
+    const f32x4 av = *(const f32x4*)(al + 4 * g);
 #pragma unroll
-      for (int h = 0; h < HB; h++) {
-        const float a = al[h];
+    for (int n = 0; n < NT; n++) o[n] *= av;
 #pragma unroll
-        for (int c = 0; c < CPT; c++) o[h][c] *= a;
+    for (int ks = 0; ks < KT / 32; ks++) {                          // (weights past nvalid are 0, rows finite)
+      if (32 * ks >= nvalid) break;
+      bf16x8 hi, lo;                                                // head r16, keys 32 ks + 8 g + e
+      const float* pw = pb + r16 * (KT + 4) + 32 * ks + 8 * g;
+#pragma unroll
+      for (int e = 0; e < 8; e += 4) {
+        const f32x4 w = *(const f32x4*)(pw + e);
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+          hi[e + i] = (__bf16)w[i];
+          lo[e + i] = (__bf16)(w[i] - (float)hi[e + i]);
+        }
       }
-      for (int j = 0; j < nvalid; j += 4) {                         // weights past nvalid are 0, rows finite
-        float kv[4][CPT];
 #pragma unroll
-        for (int jj = 0; jj < 4; jj++) {
-          const __bf16* kr = kt + (j + jj) * DP + c0;
-          if constexpr (CPT == 2) {
-            const bf16x2 v = *(const bf16x2*)kr;
-            kv[jj][0] = (float)v[0];
-            kv[jj][1] = (float)v[1];
-          } else {
-            kv[jj][0] = (float)*kr;
-          }
-        }
+      for (int n = 0; n < NT; n++) {
+        const int c = 16 * (wv + 4 * n);
+        if (c >= r) break;
+        const __bf16* kr = kt + (32 * ks + 8 * g) * DP + c + r16;    // (columns past r: the rotated part, not kept)
+        bf16x8 b;
 #pragma unroll
-        for (int h = 0; h < HB; h++) {
-          const float4 w4 = *(const float4*)(pb + h * (KT + 4) + j);
-#pragma unroll
-          for (int c = 0; c < CPT; c++)
-            o[h][c] = fmaf(w4.x, kv[0][c], fmaf(w4.y, kv[1][c], fmaf(w4.z, kv[2][c], fmaf(w4.w, kv[3][c], o[h][c]))));
-        }
+        for (int e = 0; e < 8; e++) b[e] = kr[e * DP];
+        o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lo, b, o[n], 0, 0, 0);
+        o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(hi, b, o[n], 0, 0, 0);
       }
     }
     __syncthreads();                                                // the tile and the weights are used again
@@ -188,20 +183,22 @@ __global__ void __launch_bounds__(256) latent_dec_k(const __bf16* __restrict__ q
       }
     }
   }
-  if (!mine) return;
 #pragma unroll
-  for (int h = 0; h < HB; h++) {
+  for (int i = 0; i < 4; i++) {
+    const int h = 4 * g + i;
     if (h >= nh) break;
     const int64_t th = (int64_t)t * H + h0 + h;
-    if (nsplit > 1) {
-      float* pp = part + (th * nsplit + zs) * (r + 2) + c0;
-#pragma unroll
-      for (int c = 0; c < CPT; c++) pp[c] = o[h][c];
-    } else {
-      float f = with_sink(mred[h], lred[h], sink, h0 + h);
+    float f = 1.f;
+    if (nsplit == 1) {
+      f = with_sink(mred[h], lred[h], sink, h0 + h);
       if (gate) f *= 1.0f / (1.0f + expf(-(float)gate[(int64_t)t * g_st + h0 + h]));
+    }
 #pragma unroll
-      for (int c = 0; c < CPT; c++) out[th * r + c0 + c] = (__bf16)(o[h][c] * f);
+    for (int n = 0; n < NT; n++) {
+      const int c = 16 * (wv + 4 * n) + r16;
+      if (c >= r) continue;
+      if (nsplit > 1) part[(th * nsplit + zs) * (r + 2) + c] = o[n][i];
+      else out[th * r + c] = (__bf16)(o[n][i] * f);
     }
   }
 }
@@ -281,12 +278,13 @@ bool latent_decode_fits(int r, int dr) {
 }
 
 int latent_decode_splits(int T, int H, int max_keys) {
-  const int hb = H > 8 ? 16 : 8;
-  const int64_t blocks = (int64_t)T * ((H + hb - 1) / hb);
+  const int64_t blocks = (int64_t)T * ((H + 15) / 16);
   const int tiles = (max_keys + KT - 1) / KT + 1;
-  int ns = (int)((512 + blocks - 1) / blocks);
-  ns = ns > tiles ? tiles : ns;
-  return ns < 1 ? 1 : (ns > 64 ? 64 : ns);
+  // one workgroup per CU at a time: as many splits as give every CU one, equal numbers of tiles in each
+  int ns = (int)(256 / blocks);
+  ns = ns < 1 ? 1 : (ns > 64 ? 64 : ns);
+  const int per = (tiles + ns - 1) / ns;
+  return (tiles + per - 1) / per;
 }
 
 void latent_decode(const void* q_lat, const void* q_rot, int64_t qr_st, int64_t qr_sh, const void* rows, int bs,
@@ -294,20 +292,18 @@ void latent_decode(const void* q_lat, const void* q_rot, int64_t qr_st, int64_t 
                    const void* gate, int64_t g_st, const float* sink, void* out, float* part, int nsplit, int T, int H, int r,
                    int dr, int window, hipStream_t st) {
   if (T <= 0 || !latent_decode_fits(r, dr)) return;                 // (refused by the caller beforehand)
-  const int lds = lds_bytes(r + dr), hb = H > 8 ? 16 : 8;
-  const dim3 grid(T, (H + hb - 1) / hb, nsplit);
-#define SM_DEC(CPT, HB)                                                                                                     \
-  {                                                                                                                         \
-    (void)hipFuncSetAttribute((const void*)latent_dec_k<CPT, HB>, hipFuncAttributeMaxDynamicSharedMemorySize, lds);         \
-    latent_dec_k<CPT, HB><<<grid, 256, lds, st>>>((const __bf16*)q_lat, (const __bf16*)q_rot, qr_st, qr_sh,                 \
-                                                  (const __bf16*)rows, bs, block_tables, bt_width, seq_of, pos, scale,      \
-                                                  (const __bf16*)gate, g_st, sink, (__bf16*)out, part, H, r, dr, window);   \
+  const int lds = lds_bytes(r + dr);
+  const dim3 grid(T, (H + 15) / 16, nsplit);
+#define SM_DEC(NT)                                                                                                    \
+  {                                                                                                                   \
+    (void)hipFuncSetAttribute((const void*)latent_dec_k<NT>, hipFuncAttributeMaxDynamicSharedMemorySize, lds);        \
+    latent_dec_k<NT><<<grid, 256, lds, st>>>((const __bf16*)q_lat, (const __bf16*)q_rot, qr_st, qr_sh,                \
+                                             (const __bf16*)rows, bs, block_tables, bt_width, seq_of, pos, scale,     \
+                                             (const __bf16*)gate, g_st, sink, (__bf16*)out, part, H, r, dr, window);  \
   }
-  if (r > 256) {
-    if (hb == 16) SM_DEC(2, 16) else SM_DEC(2, 8)
-  } else {
-    if (hb == 16) SM_DEC(1, 16) else SM_DEC(1, 8)
-  }
+  if (r > 256) SM_DEC(8)
+  else if (r > 128) SM_DEC(4)
+  else SM_DEC(2)
 #undef SM_DEC
   if (nsplit > 1)
     combine_k<<<dim3(T, H, (r + 255) / 256), 256, 0, st>>>(part, (const __bf16*)gate, g_st, sink, (__bf16*)out, H, r, nsplit);

@@ -695,15 +695,17 @@ __global__ void __launch_bounds__(256) pack_queries_k(const float* __restrict__ 
 }
 
 // column j: position j below nkeep, then k0, k0 + 1, ... (past the last key: that one again).  k2 [G, TW d, nk], v2 [G, TW nk,
-// dv]; a workgroup per 64 columns of a key head, the keys turned through LDS
-template <typename E>
+// dv]; a workgroup per 64 columns of a key head and 64 channels of its keys (turned through LDS) or of its values.  V values
+// per access (4: d, dv and nk are multiples of 4)
+template <typename E, int V>
 __global__ void __launch_bounds__(256) pack_keys_k(const E* __restrict__ rows, int bs, const int32_t* __restrict__ tab,
                                                   int nkeep, int64_t k0, int nr, int nk, E* __restrict__ k2,
                                                   E* __restrict__ v2, int G, int d, int dv) {
   constexpr int TW = sizeof(E) == 2 ? 2 : 1;
+  typedef E EV __attribute__((ext_vector_type(V)));
   __shared__ E tile[64][65];
   __shared__ int64_t at[64];
-  const int j0 = blockIdx.x * 64, g = blockIdx.y, nj = min(64, nk - j0);
+  const int j0 = blockIdx.x * 64, g = blockIdx.y, nj = min(64, nk - j0), kc = (d + 63) / 64;
   const int64_t ld = (int64_t)G * (d + dv);
   if (threadIdx.x < 64) {
     const int j = min(j0 + (int)threadIdx.x, nk - 1);
@@ -711,27 +713,37 @@ __global__ void __launch_bounds__(256) pack_keys_k(const E* __restrict__ rows, i
     at[threadIdx.x] = ((int64_t)tab[p / bs] * bs + p % bs) * ld;
   }
   __syncthreads();
-  for (int c0 = 0; c0 < d; c0 += 64) {
-    const int nc = min(64, d - c0);
-    __syncthreads();
-    for (int i = threadIdx.x; i < 64 * 64; i += 256) {
+  if ((int)blockIdx.z < kc) {
+    const int c0 = 64 * blockIdx.z, nc = min(64, d - c0);
+    for (int i = V * threadIdx.x; i < 64 * 64; i += V * 256) {
       const int j = i >> 6, c = i & 63;
-      if (j < nj && c < nc) tile[j][c] = rows[at[j] + (int64_t)g * d + c0 + c];
-    }
-    __syncthreads();
-    for (int i = threadIdx.x; i < 64 * 64; i += 256) {
-      const int c = i >> 6, j = i & 63;
       if (j < nj && c < nc) {
+        const EV x = *(const EV*)(rows + at[j] + (int64_t)g * d + c0 + c);
 #pragma unroll
-        for (int w = 0; w < TW; w++) k2[((int64_t)g * TW * d + w * d + c0 + c) * nk + j0 + j] = tile[j][c];
+        for (int e = 0; e < V; e++) tile[j][c + e] = x[e];
       }
     }
-  }
-  for (int i = threadIdx.x; i < nj * dv; i += 256) {
-    const int j = i / dv, c = i - j * dv;
-    const E v = rows[at[j] + (int64_t)G * d + (int64_t)g * dv + c];
+    __syncthreads();
+    for (int i = V * threadIdx.x; i < 64 * 64; i += V * 256) {
+      const int c = i >> 6, j = i & 63;
+      if (j < nj && c < nc) {
+        EV x;
 #pragma unroll
-    for (int w = 0; w < TW; w++) v2[((int64_t)g * TW * nk + (int64_t)w * nk + j0 + j) * dv + c] = v;
+        for (int e = 0; e < V; e++) x[e] = tile[j + e][c];
+#pragma unroll
+        for (int w = 0; w < TW; w++) *(EV*)(k2 + ((int64_t)g * TW * d + w * d + c0 + c) * nk + j0 + j) = x;
+      }
+    }
+  } else {
+    const int c0 = 64 * (blockIdx.z - kc), nc = min(64, dv - c0);
+    for (int i = V * threadIdx.x; i < 64 * 64; i += V * 256) {
+      const int j = i >> 6, c = i & 63;
+      if (j < nj && c < nc) {
+        const EV x = *(const EV*)(rows + at[j] + (int64_t)G * d + (int64_t)g * dv + c0 + c);
+#pragma unroll
+        for (int w = 0; w < TW; w++) *(EV*)(v2 + ((int64_t)g * TW * nk + (int64_t)w * nk + j0 + j) * dv + c0 + c) = x;
+      }
+    }
   }
 }
 
@@ -926,10 +938,12 @@ void chunk_softmax(bool bf16, float* sc, int64_t R, int Lq, int L, int G, int re
 void pack_block(bool bf16, const float* q, int64_t tok0, int nq, const void* rows, int bs, const int32_t* tab, int nkeep,
                 int64_t k0, int nr, int nk, void* q2, void* k2, void* v2, int H, int G, int d, int dv, hipStream_t st) {
   if (nq <= 0 || nk <= 0) return;
-  const dim3 gk((nk + 63) / 64, G);
+  const dim3 gk((nk + 63) / 64, G, (d + 63) / 64 + (dv + 63) / 64);
+  const bool v4 = d % 4 == 0 && dv % 4 == 0 && nk % 4 == 0 && (uintptr_t)rows % 16 == 0;
 #define MA_PACK(E)                                                                                                  \
   pack_queries_k<E><<<nq, 256, 0, st>>>(q, tok0, nq, (E*)q2, H, G, d);                                              \
-  pack_keys_k<E><<<gk, 256, 0, st>>>((const E*)rows, bs, tab, nkeep, k0, nr, nk, (E*)k2, (E*)v2, G, d, dv)
+  if (v4) pack_keys_k<E, 4><<<gk, 256, 0, st>>>((const E*)rows, bs, tab, nkeep, k0, nr, nk, (E*)k2, (E*)v2, G, d, dv); \
+  else pack_keys_k<E, 1><<<gk, 256, 0, st>>>((const E*)rows, bs, tab, nkeep, k0, nr, nk, (E*)k2, (E*)v2, G, d, dv)
   if (bf16) { MA_PACK(__bf16); } else { MA_PACK(float); }
 #undef MA_PACK
 }
