@@ -206,40 +206,41 @@ __global__ void __launch_bounds__(1024) rms_sigmoid_gate_k(const float* __restri
 // ------------------------------------------------------------------ routing
 constexpr int kPerLane = 8;                                         // experts <= 512
 
-// one wave routes token t with the logits z[0 .. E - 1]; cs, best: LDS of 64 kPerLane values
+// one wave routes token t with the logits z[0 .. E - 1]; cs, best: LDS of 64 PER values (E <= 64 PER)
 __device__ __forceinline__ void wave_sync() {
   __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
   __builtin_amdgcn_wave_barrier();
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 }
+template <int PER>
 __device__ void route_wave(const float* z, const float* __restrict__ corr, RouteRule rule, int E, int top, int groups,
                            int keep, int32_t* __restrict__ idx, float* __restrict__ w, int64_t t, float* cs, float* best) {
   const int lane = threadIdx.x & 63;
-  float s[kPerLane], c[kPerLane];
+  float s[PER], c[PER];
   float mx = -INFINITY;
 #pragma unroll
-  for (int i = 0; i < kPerLane; i++) {
+  for (int i = 0; i < PER; i++) {
     const int e = lane + 64 * i;
     s[i] = e < E ? z[e] : -INFINITY;
     mx = fmaxf(mx, s[i]);
   }
   if (rule.sigmoid) {
 #pragma unroll
-    for (int i = 0; i < kPerLane; i++) s[i] = lane + 64 * i < E ? 1.0f / (1.0f + expf(-s[i])) : 0.f;
+    for (int i = 0; i < PER; i++) s[i] = lane + 64 * i < E ? 1.0f / (1.0f + expf(-s[i])) : 0.f;
   } else {
     mx = wave_max(mx);
     float sum = 0.f;
 #pragma unroll
-    for (int i = 0; i < kPerLane; i++) {
+    for (int i = 0; i < PER; i++) {
       s[i] = lane + 64 * i < E ? expf(s[i] - mx) : 0.f;
       sum += s[i];
     }
     const float inv = 1.0f / wave_sum(sum);
 #pragma unroll
-    for (int i = 0; i < kPerLane; i++) s[i] *= inv;
+    for (int i = 0; i < PER; i++) s[i] *= inv;
   }
 #pragma unroll
-  for (int i = 0; i < kPerLane; i++) {
+  for (int i = 0; i < PER; i++) {
     const int e = lane + 64 * i;
     c[i] = e < E ? s[i] + (corr ? corr[e] : 0.f) : -INFINITY;
     if (e < E) cs[e] = c[i];
@@ -257,9 +258,9 @@ __device__ void route_wave(const float* z, const float* __restrict__ corr, Route
       best[g] = rule.best_two && gs > 1 ? b + b2 : b;
     }
     wave_sync();
-    bool kept[kPerLane];
+    bool kept[PER];
 #pragma unroll
-    for (int i = 0; i < kPerLane; i++) {
+    for (int i = 0; i < PER; i++) {
       const int g = lane + 64 * i;
       int rank = 0;
       if (g < groups) {
@@ -270,11 +271,11 @@ __device__ void route_wave(const float* z, const float* __restrict__ corr, Route
     }
     wave_sync();
 #pragma unroll
-    for (int i = 0; i < kPerLane; i++)
+    for (int i = 0; i < PER; i++)
       if (lane + 64 * i < groups) best[lane + 64 * i] = kept[i] ? 1.f : 0.f;
     wave_sync();
 #pragma unroll
-    for (int i = 0; i < kPerLane; i++) {
+    for (int i = 0; i < PER; i++) {
       const int e = lane + 64 * i;
       if (e < E && best[e / gs] == 0.f) c[i] = -INFINITY;
     }
@@ -284,7 +285,7 @@ __device__ void route_wave(const float* z, const float* __restrict__ corr, Route
     float bv = -INFINITY;
     int be = 0x7fffffff;
 #pragma unroll
-    for (int i = 0; i < kPerLane; i++)
+    for (int i = 0; i < PER; i++)
       if (c[i] > bv) {                                              // ascending e within a lane: the first of equals stays
         bv = c[i];
         be = lane + 64 * i;
@@ -304,7 +305,7 @@ __device__ void route_wave(const float* z, const float* __restrict__ corr, Route
       w[t * top + k] = 0.f;
     }
 #pragma unroll
-    for (int i = 0; i < kPerLane; i++)
+    for (int i = 0; i < PER; i++)
       if (lane + 64 * i == be) {
         idx[t * top + k] = be;
         if (!rule.renorm) w[t * top + k] = s[i];
@@ -313,7 +314,7 @@ __device__ void route_wave(const float* z, const float* __restrict__ corr, Route
     if (rule.renorm) {                                              // the winner's score to every lane
       float sv = 0.f;
 #pragma unroll
-      for (int i = 0; i < kPerLane; i++)
+      for (int i = 0; i < PER; i++)
         if (lane + 64 * i == be) sv = s[i];
       if (lane == 0) cs[k] = 0.f;
       wave_sync();
@@ -328,23 +329,24 @@ __device__ void route_wave(const float* z, const float* __restrict__ corr, Route
   }
 }
 
+template <int PER>
 __global__ void __launch_bounds__(64) route_groups_k(const float* __restrict__ z, const float* __restrict__ corr,
                                                     RouteRule rule, int E, int top, int groups, int keep, int32_t* __restrict__ idx,
                                                     float* __restrict__ w) {
-  __shared__ float cs[64 * kPerLane];                               // corrected scores
-  __shared__ float best[64 * kPerLane];                             // per group; kept ones become 1, others 0
+  __shared__ float cs[64 * PER];                                    // corrected scores
+  __shared__ float best[64 * PER];                                  // per group; kept ones become 1, others 0
   const int64_t t = blockIdx.x;
-  route_wave(z + t * E, corr, rule, E, top, groups, keep, idx, w, t, cs, best);
+  route_wave<PER>(z + t * E, corr, rule, E, top, groups, keep, idx, w, t, cs, best);
 }
 
 // few tokens: the logits as well (f32 products of the router with the token's row, a wave per router output), then the
 // first wave routes
-template <typename E, int V>
+template <typename E, int V, int PER>
 __global__ void __launch_bounds__(1024) router_k(const E* __restrict__ h, const float* __restrict__ rw,
                                                 const float* __restrict__ corr, RouteRule rule, int W, int NE, int top,
                                                 int groups, int keep,
                                                 int32_t* __restrict__ idx, float* __restrict__ w) {
-  __shared__ float cs[64 * kPerLane], best[64 * kPerLane], z[64 * kPerLane];
+  __shared__ float cs[64 * PER], best[64 * PER], z[64 * PER];
   const int64_t t = blockIdx.x;
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, NW = blockDim.x >> 6;
   for (int e = wv; e < NE; e += NW) {
@@ -361,7 +363,7 @@ __global__ void __launch_bounds__(1024) router_k(const E* __restrict__ h, const 
     if (lane == 0) z[e] = s;
   }
   __syncthreads();
-  if (wv == 0) route_wave(z, corr, rule, NE, top, groups, keep, idx, w, t, cs, best);
+  if (wv == 0) route_wave<PER>(z, corr, rule, NE, top, groups, keep, idx, w, t, cs, best);
 }
 
 int row_threads(int W, int V) {
@@ -428,15 +430,24 @@ void rms_sigmoid_gate(bool bf16, const float* o, const void* w, const void* gate
 void route_groups(const float* z, const float* corr, RouteRule rule, int T, int E, int top, int groups, int keep,
                   int32_t* idx, float* w, hipStream_t st) {
   if (T <= 0) return;
-  route_groups_k<<<T, 64, 0, st>>>(z, corr, rule, E, top, groups, keep, idx, w);
+  if (E <= 64) route_groups_k<1><<<T, 64, 0, st>>>(z, corr, rule, E, top, groups, keep, idx, w);
+  else route_groups_k<kPerLane><<<T, 64, 0, st>>>(z, corr, rule, E, top, groups, keep, idx, w);
 }
 
 void router(bool bf16, const void* h, const float* rw, const float* corr, RouteRule rule, int T, int W, int E, int top,
             int groups, int keep, int32_t* idx, float* w, hipStream_t st) {
   if (T <= 0) return;
   const int nt = 64 * (E < 16 ? E : 16);
-#define CALL(EL, V) (router_k<EL, V><<<T, nt, 0, st>>>((const EL*)h, rw, corr, rule, W, E, top, groups, keep, idx, w))
+#define CALL_P(EL, V, P) \
+  (router_k<EL, V, P><<<T, nt, 0, st>>>((const EL*)h, rw, corr, rule, W, E, top, groups, keep, idx, w))
+#define CALL(EL, V)        \
+  if (E <= 64) {           \
+    CALL_P(EL, V, 1);      \
+  } else {                 \
+    CALL_P(EL, V, kPerLane); \
+  }
   if (bf16) { SX_V(W, CALL(__bf16, 1), CALL(__bf16, 4)) } else { SX_V(W, CALL(float, 1), CALL(float, 4)) }
+#undef CALL_P
 #undef CALL
 }
 

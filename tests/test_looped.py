@@ -831,13 +831,35 @@ def test_greedy_generation_scheduler(dev):
         assert int(eng.sched.num_free_blocks()) == 8 and int(eng.sched.num_free_slots()) == batch
 
 
+def wide_cfg():
+    """sizes that the decode kernels' matrix-core forms hold: projections over row groups, wide latent tiles, per-head
+    products"""
+    return O.config([O.delta_layer(heads=4, kv_heads=2, dim=32, vdim=32, taps=4, rank=16, grank=16, mlp=O.moe(8, 2, 32, (4, 3))),
+                     O.latent_layer(heads=9, dim=32, rot_dim=16, vdim=24, kv_rank=136, window=70, mlp=O.moe(4, 2, 32, (2, 1))),
+                     O.pair_layer(heads=4, kv_heads=1, dim=32, vdim=16, dims=32, taps=2, rheads=2, rdim=32, rank=16,
+                                  mlp=O.moe(4, 3, 64, None))], vocab=100, width=128, loop=(1, 3, 2))
+
+
+def test_decode_kernels_at_their_sizes(dev):
+    """long decoding beside other requests with the sizes of ``wide_cfg``, in both number formats"""
+    cfg = no_close_calls(wide_cfg())
+    W = calm(O.random_weights(cfg, 26))
+    P = {"a": O.random_tokens(cfg, 150, 1), "b": O.random_tokens(cfg, 70, 2), "c": O.random_tokens(cfg, 25, 3)}
+    schedule = [[("a", 100), ("b", 20)]] + [[("a", 1), ("b", 1), ("c", 1)]] * 25 + [[("a", 1), ("b", 1)]] * 25
+    for dtype in (torch.float32, torch.bfloat16):
+        got = replay(engine(cfg, W, dev, dtype), P, schedule)
+        for name, toks in P.items():
+            assert rel_err(got[name], oracle(cfg, W, toks, "wide" + name)) < TOL[dtype], name
+
+
 @pytest.mark.gpu
-def test_decode_graph_replays_equal_eager():
+@pytest.mark.parametrize("sizes", ["narrow", "wide"])
+def test_decode_graph_replays_equal_eager(sizes):
     """pure-decode steps replayed from a captured graph (padded rows on the scratch page and slot), with eager
     prompt steps and synchronisations between the replays"""
     if not torch.cuda.is_available():
         pytest.skip("no GPU")
-    cfg = std_cfg()
+    cfg = std_cfg() if sizes == "narrow" else wide_cfg()
     W = O.random_weights(cfg, 21)
     P = {"a": O.random_tokens(cfg, 90, 1), "b": O.random_tokens(cfg, 40, 2), "c": O.random_tokens(cfg, 75, 3)}
     schedule = [[("a", 60), ("b", 20)]] + [[("a", 1), ("b", 1)]] * 10 + [[("c", 66)]] + \
